@@ -50,7 +50,8 @@ def weight_bytes(model, itemsize: int = 2) -> int:
 def kv_bytes(model, context: float, itemsize: int = 2) -> float:
     """Bytes of cache that a request with `context` tokens has a decode step read: what every cache
     layer keeps per token (`Model.cache_elements_per_token`), over the keys it still holds."""
-    return sum(itemsize * n * (context if w is None else min(context, w)) for n, w in model.cache_elements_per_token())
+    from serve_amd.cache.retention import mean_seen
+    return sum(itemsize * n * mean_seen(rule, context) for n, rule in model.cache_elements_per_token())
 
 
 def prefill_flops(model, T: int) -> float:

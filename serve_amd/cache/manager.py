@@ -6,8 +6,9 @@ request and frees only when a request completes (serve/kv_cache_paged.py:17-80).
 ids back from the device to free them (:72) and has no check for an empty pool (:57-60).  Here
 the table is mirrored on the host, allocation is all-or-nothing, and layers are put in
 *groups*: layers that keep all keys form one group, layers that keep a window of W keys
-another; each group has its own pool and its own block table per request, and a windowed
-group gives pages back as soon as the window has passed them.
+another, layers that see chunks of n positions a third (`cache.retention`); each group has its
+own pool and its own block table per request, and a group that keeps a window or a chunk gives
+pages back as soon as no later token can see them.
 
 A page id means the same row in the page tensors of every layer of its group.  Freed pages
 are reused last-in first-out, so a page given back is the next one handed out.
@@ -19,7 +20,10 @@ from typing import Dict, List, Optional, Sequence
 
 import numpy as np
 
-FREED = -1      # block-table entry of a page that the window has passed
+from . import retention
+from .retention import Retention
+
+FREED = -1      # block-table entry of a page that the window or the chunk has passed
 
 
 class CacheError(RuntimeError):
@@ -68,18 +72,18 @@ class _Request:
 class CacheManager:
     """Pages and block tables for `len(windows)` groups, and `max_requests` state slots.
 
-    `windows[g]` is None for a group that keeps every key, or W for one that keeps the last W.
+    `windows[g]` is group g's retention rule: None for one that keeps every key, W for one that keeps the last W,
+    `Chunks(n)` for one that keeps the current run of n positions.
     """
 
-    def __init__(self, windows: Sequence[Optional[int]], num_pages: Sequence[int], page_size: int,
+    def __init__(self, windows: Sequence[Retention], num_pages: Sequence[int], page_size: int,
                  max_requests: int, max_pages_per_request: int):
         if len(windows) != len(num_pages):
             raise ValueError("one pool size per group is needed")
         if page_size <= 0 or max_requests <= 0 or max_pages_per_request <= 0:
             raise ValueError("page_size, max_requests and max_pages_per_request must be positive")
         for w in windows:
-            if w is not None and w <= 0:
-                raise ValueError("a window must be positive")
+            retention.check(w)
         self.windows = list(windows)
         self.page_size = page_size
         self.max_requests = max_requests
@@ -128,12 +132,13 @@ class CacheManager:
         """Per group: the most pages a request holds at any time on its way to `n_tokens` tokens
         when it is fed in portions of at most `portion` tokens and trimmed after every step.  A
         group that keeps every key needs the pages of all its tokens; a group that keeps a window
-        of W keys never holds more than the window, one portion and the page their first key
-        shares with keys that have gone."""
+        of W keys (or a chunk of as many) never holds more than that, one portion and the page their
+        first key shares with keys that have gone."""
         ps = self.page_size
         whole = -(-n_tokens // ps)
         out = []
-        for w in self.windows:
+        for rule in self.windows:
+            w = retention.reach(rule)
             if w is None:
                 out.append(whole)
             else:
@@ -142,11 +147,7 @@ class CacheManager:
 
     def _first_live_index(self, group: int, n_tokens: int) -> int:
         """Index of the first page a query at position >= n_tokens can still see."""
-        w = self.windows[group]
-        if w is None:
-            return 0
-        first_key = max(0, n_tokens - w + 1)
-        return first_key // self.page_size
+        return retention.first_seen(self.windows[group], n_tokens) // self.page_size
 
     def pages_needed(self, req_id, n_tokens: int) -> List[int]:
         """Per group: pages that `ensure(req_id, n_tokens)` would take (0 for an unknown request
@@ -196,7 +197,7 @@ class CacheManager:
         return True
 
     def trim(self, req_id, n_tokens_done: int) -> int:
-        """Give back the pages of windowed groups that no query at position >= n_tokens_done can
+        """Give back the pages of groups with a window or a chunk that no query at position >= n_tokens_done can
         see.  Returns the number of pages freed."""
         r = self._requests[req_id]
         freed = 0

@@ -14,15 +14,17 @@ from typing import List, Optional, Sequence
 import torch
 
 from ..parts.base import LayerCache, Runtime, StateRequest, TokenCacheRequest
+from . import retention
+from .retention import Retention
 
 
-def group_windows(requests: Sequence[Optional[TokenCacheRequest]]) -> List[Optional[int]]:
+def group_windows(requests: Sequence[Optional[TokenCacheRequest]]) -> List[Retention]:
     """The distinct retention rules of the model's cache layers, full retention first."""
-    seen: List[Optional[int]] = []
+    seen: List[Retention] = []
     for r in requests:
-        if r is not None and r.window not in seen:
-            seen.append(r.window)
-    seen.sort(key=lambda w: (w is not None, w or 0))
+        if r is not None and r.retention not in seen:
+            seen.append(r.retention)
+    seen.sort(key=retention.sort_key)
     return seen
 
 
@@ -30,7 +32,7 @@ def _itemsize(dtype: torch.dtype) -> int:
     return torch.empty((), dtype=dtype).element_size()
 
 
-def bytes_per_page(requests: Sequence[Optional[TokenCacheRequest]], windows: Sequence[Optional[int]],
+def bytes_per_page(requests: Sequence[Optional[TokenCacheRequest]], windows: Sequence[Retention],
                    page_size: int, dtype: torch.dtype) -> List[int]:
     """Per group: bytes that one page id costs over all layers of the group (`dtype` is the
     activation dtype, which a cache tensor without a dtype of its own takes)."""
@@ -38,13 +40,13 @@ def bytes_per_page(requests: Sequence[Optional[TokenCacheRequest]], windows: Seq
     for r in requests:
         if r is not None:
             for t in r.tensors:
-                out[windows.index(r.window)] += t.elements_per_token() * page_size * _itemsize(t.dtype or dtype)
+                out[windows.index(r.retention)] += t.elements_per_token() * page_size * _itemsize(t.dtype or dtype)
     return out
 
 
 class CacheStorage:
     def __init__(self, rt: Runtime, cache_requests: Sequence[Optional[TokenCacheRequest]],
-                 state_requests: Sequence[Optional[StateRequest]], windows: Sequence[Optional[int]],
+                 state_requests: Sequence[Optional[StateRequest]], windows: Sequence[Retention],
                  num_pages: Sequence[int], page_size: int, max_requests: int, poison: bool = False):
         """`poison` (debugging): pages hold NaN until a token is stored in them, and again once they
         are given back (`poison_pages`): a kernel that reads a key it must not see then shows in the
@@ -54,7 +56,7 @@ class CacheStorage:
         for cr, sr in zip(cache_requests, state_requests):
             lc = LayerCache(page_size=page_size)
             if cr is not None:
-                g = list(windows).index(cr.window)
+                g = list(windows).index(cr.retention)
                 lc.group = g
                 names = [t.name for t in cr.tensors]
                 if len(set(names)) != len(names):

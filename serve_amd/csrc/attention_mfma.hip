@@ -83,7 +83,7 @@ __device__ __forceinline__ void attention_tile(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ block_table, int max_pages, const int* __restrict__ ctx_len, int Hq, int Hk,
-    int page_size, int page_shift, float scale_log2e, int window, int num_splits,
+    int page_size, int page_shift, float scale_log2e, int window, int chunk, int num_splits,
     float* __restrict__ part_o, float* __restrict__ part_ml, const float* __restrict__ sinks) {
   constexpr int NT = 1;                                     // column tiles of 16 rows per wave
   const int lane = threadIdx.x & 63;
@@ -98,8 +98,7 @@ __device__ __forceinline__ void attention_tile(
   const int j_lo = r0 / G;
   const int j_hi = min(rows_total - 1, r0 + 16 * NT - 1) / G;
   const int hi_key = ctx_before + j_hi;
-  int lo_key = 0;
-  if (window > 0) lo_key = max(0, ctx_before + j_lo - window + 1);
+  const int lo_key = first_seen_key(ctx_before + j_lo, window, chunk);
   const int kb_lo = lo_key >> 5;
   const int kb_hi = hi_key >> 5;
   const int per = (kb_hi - kb_lo + num_splits) / num_splits;   // ceil((kb_hi - kb_lo + 1) / splits)
@@ -107,13 +106,13 @@ __device__ __forceinline__ void attention_tile(
   const int b0 = __builtin_amdgcn_readfirstlane(kb_lo + sp * per);
   const int b1 = __builtin_amdgcn_readfirstlane(min(kb_hi + 1, b0 + per));
   // blocks full_lo .. full_hi are visible as a whole to every row of the tile and need no mask:
-  // their last key is at most the first row's position, their first key inside the last row's window
+  // their last key is at most the first row's position, their first key not before the last row's first
   const int full_hi = __builtin_amdgcn_readfirstlane((ctx_before + j_lo - 31) >> 5);
-  const int full_lo = window > 0 ? __builtin_amdgcn_readfirstlane(((ctx_before + j_hi - window) >> 5) + 1) : 0;
+  const int full_lo = __builtin_amdgcn_readfirstlane((first_seen_key(ctx_before + j_hi, window, chunk) + 31) >> 5);
   const int* bt = block_table + (size_t)seg * max_pages;
 
   // this lane's query column in each column tile
-  int qpos[NT], tok[NT], head[NT];
+  int qpos[NT], qlo[NT], tok[NT], head[NT];
   bool rvalid[NT];
   Frag qf[NT][DC];
 #pragma unroll
@@ -125,6 +124,7 @@ __device__ __forceinline__ void attention_tile(
     tok[n] = q_begin + j;
     head[n] = hk * G + (rowc - j * G);
     qpos[n] = ctx_before + j;
+    qlo[n] = first_seen_key(qpos[n], window, chunk);
     const bf16_t* qp = q + (size_t)tok[n] * q_stride + (size_t)head[n] * HD;
 #pragma unroll
     for (int dc = 0; dc < DC; ++dc) {
@@ -302,7 +302,7 @@ __device__ __forceinline__ void attention_tile(
           float x = s[t][n][r];
           if (MASKED) {
             const int key = key0 + 8 * g + 4 * t + r;
-            const bool vis = key <= qpos[n] && (window <= 0 || key > qpos[n] - window);
+            const bool vis = key <= qpos[n] && key >= qlo[n];
             x = vis ? x : -INFINITY;
           }
           v[t][r] = x;
@@ -414,7 +414,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ block_table, int max_pages, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_len, int Hq, int Hk, int page_size, int page_shift, float scale_log2e,
-    int window, int num_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
+    int window, int chunk, int num_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
     const float* __restrict__ sinks) {
   const int w = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int hk = blockIdx.y;
@@ -423,7 +423,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
   const int q_begin = cu_q[seg];
   const int q_len = cu_q[seg + 1] - q_begin;
   attention_tile<PM>(w, seg, hk, sp, q_begin, q_len, q, q_stride, out, k_pages, v_pages, block_table, max_pages,
-                     ctx_len, Hq, Hk, page_size, page_shift, scale_log2e, window, num_splits, part_o, part_ml, sinks);
+                     ctx_len, Hq, Hk, page_size, page_shift, scale_log2e, window, chunk, num_splits, part_o, part_ml, sinks);
 }
 
 // The same for short contexts: the WS waves of a workgroup take the WS parts of the key range of one
@@ -438,7 +438,7 @@ __global__ __launch_bounds__(64 * WG_SPLITS) void paged_attention_mfma_wg_kernel
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ block_table, int max_pages, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_len, int Hq, int Hk, int page_size, int page_shift, float scale_log2e,
-    int window, const float* __restrict__ sinks) {
+    int window, int chunk, const float* __restrict__ sinks) {
   __shared__ float part_o[WG_SPLITS * 16 * HD];
   __shared__ float part_ml[WG_SPLITS * 16 * 2];
   const int wave = threadIdx.x >> 6;
@@ -447,7 +447,7 @@ __global__ __launch_bounds__(64 * WG_SPLITS) void paged_attention_mfma_wg_kernel
   const int q_begin = cu_q[seg];
   const int q_len = cu_q[seg + 1] - q_begin;
   attention_tile<PM, true>(0, seg, hk, wave, q_begin, q_len, q, q_stride, out, k_pages, v_pages, block_table,
-                           max_pages, ctx_len, Hq, Hk, page_size, page_shift, scale_log2e, window, WG_SPLITS,
+                           max_pages, ctx_len, Hq, Hk, page_size, page_shift, scale_log2e, window, chunk, WG_SPLITS,
                            part_o, part_ml, nullptr);
   __syncthreads();
   if (wave != 0) return;
@@ -513,7 +513,7 @@ __global__ __launch_bounds__(64 * WG_SPLITS) void paged_attention_mfma_wg_kernel
 // rescaled only when a maximum has moved, and page addresses that are a constant plus a product.
 //
 // The work per stage is the same straight line of code for every wave and stage: a block that is
-// partly or wholly invisible to the tile (the causal edge, the window's edge, beyond the tile's
+// partly or wholly invisible to the tile (the causal edge, the window's or chunk's edge, beyond the tile's
 // last key) has its scores masked under a branch that touches nothing else, and contributes
 // p = 0.  A branch around the matrix products themselves would make the compiler copy O at every
 // stage.
@@ -559,7 +559,7 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ block_table, int max_pages, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_len, int Hq, int Hk, int page_size, int page_shift, float scale_log2e,
-    int window, int num_splits, int pair, float* __restrict__ part_o, float* __restrict__ part_ml,
+    int window, int chunk, int num_splits, int pair, float* __restrict__ part_o, float* __restrict__ part_ml,
     const float* __restrict__ sinks) {
   using S = PromptShape<KW>;
   constexpr int TW = S::TW, KB = S::KB, NT = 2, PT = S::PER_THREAD;
@@ -732,7 +732,7 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
     // the workgroup's range of stages, and this split's part of it
     const int r0g = group * (32 * TW);
     const int hi_key_g = ctx_before + min(rows_total - 1, r0g + 32 * TW - 1) / G;
-    const int lo_key_g = window > 0 ? max(0, ctx_before + r0g / G - window + 1) : 0;
+    const int lo_key_g = first_seen_key(ctx_before + r0g / G, window, chunk);
     lo_visible = lo_key_g;
     const int sb_lo = lo_key_g / S::KEYS;
     const int sb_hi = hi_key_g / S::KEYS;
@@ -747,9 +747,9 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
     const int j_hi = min(rows_total - 1, r0 + 31) / G;
     // blocks full_lo .. full_hi are visible as a whole to every row of the tile
     const int full_hi = __builtin_amdgcn_readfirstlane((ctx_before + j_lo - 31) >> 5);
-    const int full_lo = window > 0 ? __builtin_amdgcn_readfirstlane(((ctx_before + j_hi - window) >> 5) + 1) : 0;
+    const int full_lo = __builtin_amdgcn_readfirstlane((first_seen_key(ctx_before + j_hi, window, chunk) + 31) >> 5);
 
-    int qpos[NT], tok[NT], head[NT];
+    int qpos[NT], qlo[NT], tok[NT], head[NT];
     bool rvalid[NT];
     Frag qf[NT][DC];
     float m[NT], m_raw[NT];
@@ -764,6 +764,7 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
       tok[n] = q_begin + j;
       head[n] = hk * G + (rowc - j * G);
       qpos[n] = ctx_before + j;
+      qlo[n] = first_seen_key(qpos[n], window, chunk);
       const bf16_t* qp = q + (size_t)tok[n] * q_stride + (size_t)head[n] * HD;
 #pragma unroll
       for (int dc = 0; dc < DC; ++dc) {
@@ -823,7 +824,7 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
 #pragma unroll
               for (int r = 0; r < 4; ++r) {
                 const int key = ((kb + h) << 5) + 8 * g + 4 * t + r;
-                const bool vis = key <= qpos[n] && (window <= 0 || key > qpos[n] - window);
+                const bool vis = key <= qpos[n] && key >= qlo[n];
                 s[h][t][n][r] = vis ? s[h][t][n][r] : -INFINITY;
               }
       }
@@ -1005,7 +1006,7 @@ template <int KW, int PM>
 static int launch_prompt(dim3 grid, hipStream_t stream, const bf16_t* q, int q_stride, bf16_t* out,
                          const bf16_t* k_pages, const bf16_t* v_pages, const int* block_table, int max_pages,
                          const int* cu_q, const int* ctx_len, int Hq, int Hk, int page_size, int page_shift,
-                         float scale_log2e, int window, int num_splits, int pair, float* part_o, float* part_ml,
+                         float scale_log2e, int window, int chunk, int num_splits, int pair, float* part_o, float* part_ml,
                          const float* sinks) {
   constexpr int lds = PromptShape<KW>::LDS_BYTES;
   static bool sized = false;          // more than 64 KB of LDS has to be asked for, once per kernel
@@ -1017,7 +1018,7 @@ static int launch_prompt(dim3 grid, hipStream_t stream, const bf16_t* q, int q_s
   }
   hipLaunchKernelGGL((prompt_attention_kernel<KW, PM>), grid, dim3(512), lds, stream, q, q_stride, out, k_pages,
                      v_pages, block_table, max_pages, cu_q, ctx_len, Hq, Hk, page_size, page_shift, scale_log2e,
-                     window, num_splits, pair, part_o, part_ml, sinks);
+                     window, chunk, num_splits, pair, part_o, part_ml, sinks);
   return 0;
 }
 
@@ -1073,12 +1074,12 @@ extern "C" int sa_attention_mfma_head_dim() { return HD; }
 extern "C" int sa_paged_attention_mfma(const void* q, int q_stride, void* out, const void* k_pages,
                                        const void* v_pages, const int* block_table, int max_pages,
                                        const int* cu_q, const int* ctx_len, int B, int T, int max_q_len,
-                                       int Hq, int Hk, int D, int page_size, float scale, int window,
+                                       int Hq, int Hk, int D, int page_size, float scale, int window, int chunk,
                                        int num_splits, float* part_o, float* part_ml, int in_workgroup,
                                        const float* sinks, hipStream_t stream) {
   if (T <= 0 || B <= 0) return 0;
   if (D != HD || Hq <= 0 || Hk <= 0 || Hq % Hk || page_size <= 0 || (page_size & 3) || max_pages <= 0 ||
-      max_q_len <= 0 || num_splits < 1 || num_splits > 64 || (q_stride & 7))
+      max_q_len <= 0 || num_splits < 1 || num_splits > 64 || (q_stride & 7) || (window > 0 && chunk > 0))
     return SA_ERR_ARG;
   if (num_splits > 1 && (!part_o || !part_ml)) return SA_ERR_ARG;
   if ((long long)B * num_splits > 65535 || Hk > 65535) return SA_ERR_ARG;
@@ -1099,7 +1100,7 @@ extern "C" int sa_paged_attention_mfma(const void* q, int q_stride, void* out, c
   hipLaunchKernelGGL((paged_attention_mfma_wg_kernel<PM>), grid, block, 0, stream,                     \
                      (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages,                 \
                      (const bf16_t*)v_pages, block_table, max_pages, cu_q, ctx_len, Hq, Hk, page_size, \
-                     page_shift, scale_log2e, window, sinks)
+                     page_shift, scale_log2e, window, chunk, sinks)
     if (pm == 2) GO(2);
     else if (pm == 1) GO(1);
     else GO(0);
@@ -1115,7 +1116,7 @@ extern "C" int sa_paged_attention_mfma(const void* q, int q_stride, void* out, c
   hipLaunchKernelGGL((paged_attention_mfma_kernel<PM>), grid, block, 0, stream,                        \
                      (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages,                 \
                      (const bf16_t*)v_pages, block_table, max_pages, cu_q, ctx_len, Hq, Hk, page_size, \
-                     page_shift, scale_log2e, window, num_splits, part_o, part_ml, sinks)
+                     page_shift, scale_log2e, window, chunk, num_splits, part_o, part_ml, sinks)
     if (pm == 2) GO(2);
     else if (pm == 1) GO(1);
     else GO(0);
@@ -1137,7 +1138,7 @@ extern "C" int sa_paged_attention_mfma(const void* q, int q_stride, void* out, c
 #define GO(KW, PM)                                                                                       \
   rc = launch_prompt<KW, PM>(grid, stream, (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages, \
                              (const bf16_t*)v_pages, block_table, max_pages, cu_q, ctx_len, Hq, Hk, page_size, \
-                             page_shift, scale_log2e, window, num_splits, pair, part_o, part_ml, sinks)
+                             page_shift, scale_log2e, window, chunk, num_splits, pair, part_o, part_ml, sinks)
     if (kw == 2 && pm == 1) GO(2, 1);
     else if (kw == 2) GO(2, 0);
     else if (pm == 1) GO(4, 1);

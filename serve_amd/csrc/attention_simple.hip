@@ -4,7 +4,8 @@
 // The first is the general form: any head_dim up to 640, any head counts, any page size, any mix of
 // prompt portions and single tokens in one launch.  Formulas as in serve/kernels/attn_prefill.py:56-72,205 and attn_decode.py:99-111,236:
 // scores = q.k * scale, key j visible to the query at absolute position p iff j <= p (and
-// p - j < window when a window is set), online softmax (m, l, O), O / l at the end.  Query head
+// p - j < window when a window is set; j / chunk == p / chunk when a chunk is: at most one of the two),
+// online softmax (m, l, O), O / l at the end.  Query head
 // h reads KV head h / (Hq / Hk).  With `sinks` (fp32 [Hq], or null) the softmax of head h has one more
 // term exp(sinks[h]) in its denominator (sinks[h] as it is stored: `scale` does not apply to it), which takes
 // weight away from the keys and adds nothing to the output: it joins l
@@ -23,7 +24,7 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
     const TA* __restrict__ q, int q_stride, TA* __restrict__ out, const TC* __restrict__ k_pages,
     const TC* __restrict__ v_pages, const int* __restrict__ block_table, int max_pages,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_len, const int* __restrict__ seg_of_token,
-    int Hq, int Hk, int D, int page_size, float scale, int window, int t0, const float* __restrict__ sinks) {
+    int Hq, int Hk, int D, int page_size, float scale, int window, int chunk, int t0, const float* __restrict__ sinks) {
   __shared__ float qs[SA_MAX_D];
   __shared__ float ps[SA_WAVE];
   __shared__ int vbase_page[SA_WAVE];
@@ -42,8 +43,7 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
   for (int i = lane; i < D; i += SA_WAVE) qs[i] = to_float(qrow[i]);
   __syncthreads();
 
-  int lo = 0;
-  if (window > 0 && qpos - window + 1 > 0) lo = qpos - window + 1;
+  const int lo = first_seen_key(qpos, window, chunk);
   const int hi = qpos;  // inclusive
 
   float m = -INFINITY, l = 0.f;
@@ -116,7 +116,7 @@ __global__ __launch_bounds__(256) void paged_attention_tiled_f32_kernel(
     const float* __restrict__ q, int q_stride, float* __restrict__ out, const float* __restrict__ k_pages,
     const float* __restrict__ v_pages, const int* __restrict__ block_table, int max_pages,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_len, int Hq, int Hk, int page_size, float scale,
-    int window, int num_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
+    int window, int chunk, int num_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
     const float* __restrict__ sinks) {
   constexpr int D = DV * 16;
   constexpr int LD = D + 4;                       // row length in LDS: keeps 16-byte alignment, spreads banks
@@ -151,16 +151,17 @@ __global__ __launch_bounds__(256) void paged_attention_tiled_f32_kernel(
     *reinterpret_cast<float4*>(Qs + r * LD + c4 * 4) =
         *reinterpret_cast<const float4*>(q + (size_t)(q_begin + j) * q_stride + (size_t)(g * G + gi) * D + c4 * 4);
   }
-  int qpos[4];
+  int qpos[4], qlo[4];
   bool rvalid[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int row = r0 + tr * 4 + r;
     rvalid[r] = row < rows_total;
     qpos[r] = ctx_before + min(row, rows_total - 1) / G;
+    qlo[r] = first_seen_key(qpos[r], window, chunk);
   }
   const int hi = ctx_before + min(r0 + TL_ROWS - 1, rows_total - 1) / G;          // last key any row of the tile sees
-  const int lo = window > 0 ? max(0, ctx_before + r0 / G - window + 1) : 0;      // first key any row sees
+  const int lo = first_seen_key(ctx_before + r0 / G, window, chunk);              // first key any row sees
 
   float m[4], l[4], acc[4][DV];
 #pragma unroll
@@ -245,7 +246,7 @@ __global__ __launch_bounds__(256) void paged_attention_tiled_f32_kernel(
 #pragma unroll
       for (int c = 0; c < 4; ++c) {
         const int key = kb + tc + 16 * c;
-        const bool vis = key <= qpos[r] && (window <= 0 || key > qpos[r] - window);
+        const bool vis = key <= qpos[r] && key >= qlo[r];
         s[r][c] = vis ? s[r][c] * scale : -INFINITY;
         mx = fmaxf(mx, s[r][c]);
       }
@@ -351,7 +352,7 @@ __global__ __launch_bounds__(64) void paged_attention_merge_f32_kernel(const flo
 template <int DV>
 static int launch_tiled(const void* q, int q_stride, void* out, const void* k_pages, const void* v_pages,
                         const int* block_table, int max_pages, const int* cu_q, const int* ctx_len, int B,
-                        int max_q_len, int Hq, int Hk, int page_size, float scale, int window, int num_splits,
+                        int max_q_len, int Hq, int Hk, int page_size, float scale, int window, int chunk, int num_splits,
                         float* part_o, float* part_ml, const float* sinks, hipStream_t stream) {
   constexpr int D = DV * 16;
   const size_t lds = (size_t)(3 * 64 * (D + 4) + 64 * 68) * sizeof(float);
@@ -363,7 +364,7 @@ static int launch_tiled(const void* q, int q_stride, void* out, const void* k_pa
   dim3 grid((unsigned)(items * Hk), B * num_splits), block(256);
   hipLaunchKernelGGL((paged_attention_tiled_f32_kernel<DV>), grid, block, lds, stream, (const float*)q, q_stride,
                      (float*)out, (const float*)k_pages, (const float*)v_pages, block_table, max_pages, cu_q,
-                     ctx_len, Hq, Hk, page_size, scale, window, num_splits, part_o, part_ml, sinks);
+                     ctx_len, Hq, Hk, page_size, scale, window, chunk, num_splits, part_o, part_ml, sinks);
   SA_LAUNCH_CHECK();
   return 0;
 }
@@ -387,7 +388,7 @@ __global__ __launch_bounds__(64) void paged_attention_decode_f32_kernel(
     const float* __restrict__ q, int q_stride, float* __restrict__ out, const float* __restrict__ k_pages,
     const float* __restrict__ v_pages, const int* __restrict__ block_table, int max_pages,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_len, int Hq, int Hk, int page_size, float scale,
-    int window, int num_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
+    int window, int chunk, int num_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
     const float* __restrict__ sinks) {
   constexpr int D = DV * 16;
   constexpr int NA = (D + 63) / 64;               // dims per lane in the product with V
@@ -403,7 +404,7 @@ __global__ __launch_bounds__(64) void paged_attention_decode_f32_kernel(
   const int t = cu_q[seg];                        // the segment's one token
   const int qpos = ctx_len[seg] - 1;
   const int* bt = block_table + (size_t)seg * max_pages;
-  const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
+  const int lo = first_seen_key(qpos, window, chunk);
   const int hi = qpos;
 
   // this lane's quarter of the queries (a head beyond the group repeats the last and is not written)
@@ -538,7 +539,7 @@ __global__ __launch_bounds__(64) void paged_attention_decode_f32_kernel(
 template <int DV>
 static int launch_decode_f32(const void* q, int q_stride, void* out, const void* k_pages, const void* v_pages,
                              const int* block_table, int max_pages, const int* cu_q, const int* ctx_len, int B,
-                             int Hq, int Hk, int page_size, float scale, int window, int num_splits, float* part_o,
+                             int Hq, int Hk, int page_size, float scale, int window, int chunk, int num_splits, float* part_o,
                              float* part_ml, const float* sinks, hipStream_t stream) {
   const int G = Hq / Hk;
   const int gr = G >= 3 ? 4 : G;                  // heads per wave: 1, 2 or 4
@@ -548,7 +549,7 @@ static int launch_decode_f32(const void* q, int q_stride, void* out, const void*
 #define GO(GR)                                                                                                    \
   hipLaunchKernelGGL((paged_attention_decode_f32_kernel<DV, GR>), grid, block, 0, stream, (const float*)q,        \
                      q_stride, (float*)out, (const float*)k_pages, (const float*)v_pages, block_table, max_pages, \
-                     cu_q, ctx_len, Hq, Hk, page_size, scale, window, num_splits, part_o, part_ml, sinks)
+                     cu_q, ctx_len, Hq, Hk, page_size, scale, window, chunk, num_splits, part_o, part_ml, sinks)
   if (gr == 1) GO(1);
   else if (gr == 2) GO(2);
   else GO(4);
@@ -567,18 +568,19 @@ static int launch_decode_f32(const void* q, int q_stride, void* out, const void*
 extern "C" int sa_paged_attention_decode_f32(const void* q, int q_stride, void* out, const void* k_pages,
                                              const void* v_pages, const int* block_table, int max_pages,
                                              const int* cu_q, const int* ctx_len, int B, int first_token, int Hq,
-                                             int Hk, int D, int page_size, float scale, int window, int num_splits,
-                                             float* part_o, float* part_ml, const float* sinks, hipStream_t stream) {
+                                             int Hk, int D, int page_size, float scale, int window, int chunk,
+                                             int num_splits, float* part_o, float* part_ml, const float* sinks, hipStream_t stream) {
   if (B <= 0) return 0;
   if (Hq <= 0 || Hk <= 0 || Hq % Hk || D <= 0 || D > 128 || (D & 15) || page_size <= 0 || (page_size & 3) ||
-      max_pages <= 0 || (q_stride & 3) || num_splits < 1 || num_splits > 64 || first_token < 0)
+      max_pages <= 0 || (q_stride & 3) || num_splits < 1 || num_splits > 64 || first_token < 0 ||
+      (window > 0 && chunk > 0))
     return SA_ERR_ARG;
   if (num_splits > 1 && (!part_o || !part_ml)) return SA_ERR_ARG;
   int rc = SA_ERR_ARG;
 #define GO(DV)                                                                                                   \
   case DV:                                                                                                       \
     rc = launch_decode_f32<DV>(q, q_stride, out, k_pages, v_pages, block_table, max_pages, cu_q, ctx_len, B, Hq, \
-                               Hk, page_size, scale, window, num_splits, part_o, part_ml, sinks, stream);        \
+                               Hk, page_size, scale, window, chunk, num_splits, part_o, part_ml, sinks, stream); \
     break
   switch (D / 16) {
     GO(1);
@@ -609,18 +611,18 @@ extern "C" int sa_paged_attention_tiled_f32(const void* q, int q_stride, void* o
                                             const void* v_pages, const int* block_table, int max_pages,
                                             const int* cu_q, const int* ctx_len, int B, int T, int max_q_len,
                                             int Hq, int Hk, int D, int page_size, float scale, int window,
-                                            int num_splits, float* part_o, float* part_ml, const float* sinks,
+                                            int chunk, int num_splits, float* part_o, float* part_ml, const float* sinks,
                                             hipStream_t stream) {
   if (B <= 0 || max_q_len <= 0 || T <= 0) return 0;
   if (Hq <= 0 || Hk <= 0 || Hq % Hk || D <= 0 || D > 128 || (D & 15) || page_size <= 0 || (page_size & 3) ||
-      max_pages <= 0 || (q_stride & 3) || num_splits < 1 || num_splits > 64)
+      max_pages <= 0 || (q_stride & 3) || num_splits < 1 || num_splits > 64 || (window > 0 && chunk > 0))
     return SA_ERR_ARG;
   if (num_splits > 1 && (!part_o || !part_ml)) return SA_ERR_ARG;
   int rc = SA_ERR_ARG;
 #define GO(DV)                                                                                                  \
   case DV:                                                                                                      \
     rc = launch_tiled<DV>(q, q_stride, out, k_pages, v_pages, block_table, max_pages, cu_q, ctx_len, B,         \
-                          max_q_len, Hq, Hk, page_size, scale, window, num_splits, part_o, part_ml, sinks,     \
+                          max_q_len, Hq, Hk, page_size, scale, window, chunk, num_splits, part_o, part_ml, sinks, \
                           stream);                                                                              \
     break
   switch (D / 16) {
@@ -645,10 +647,11 @@ extern "C" int sa_paged_attention_simple(const void* q, int q_stride, void* out,
                                          const void* k_pages, const void* v_pages, int cache_dtype,
                                          const int* block_table, int max_pages, const int* cu_q,
                                          const int* ctx_len, const int* seg_of_token, int T, int Hq,
-                                         int Hk, int D, int page_size, float scale, int window,
+                                         int Hk, int D, int page_size, float scale, int window, int chunk,
                                          const float* sinks, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (Hq <= 0 || Hk <= 0 || Hq % Hk || D <= 0 || D > SA_MAX_D || page_size <= 0 || max_pages <= 0)
+  if (Hq <= 0 || Hk <= 0 || Hq % Hk || D <= 0 || D > SA_MAX_D || page_size <= 0 || max_pages <= 0 ||
+      (window > 0 && chunk > 0))
     return SA_ERR_ARG;
   if (T > 65535 * 16) return SA_ERR_ARG;
   // grid.y is limited to 65535: long steps are launched in slices of tokens
@@ -660,7 +663,7 @@ extern "C" int sa_paged_attention_simple(const void* q, int q_stride, void* out,
   hipLaunchKernelGGL((paged_attention_simple_kernel<TA, TC>), grid, block, 0, stream,                \
                      (const TA*)q, q_stride, (TA*)out, (const TC*)k_pages, (const TC*)v_pages,       \
                      block_table, max_pages, cu_q, ctx_len, seg_of_token, Hq, Hk, D, page_size,     \
-                     scale, window, t0, sinks)
+                     scale, window, chunk, t0, sinks)
     if (act_dtype == SA_F32 && cache_dtype == SA_F32) GO(float, float);
     else if (act_dtype == SA_BF16 && cache_dtype == SA_BF16) GO(bf16_t, bf16_t);
     else return SA_ERR_UNSUPPORTED;

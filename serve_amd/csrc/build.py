@@ -50,6 +50,7 @@ SOURCES: Dict[str, str] = {
     "moe": "moe.hip",
     "qk_norm": "qk_norm.hip",
     "recurrent_scan": "recurrent_scan.hip",
+    "gated_average": "gated_average.hip",
     "stream_ops": "stream_ops.hip",
 }
 # what a library is linked with beside the HIP runtime

@@ -86,6 +86,32 @@ __device__ __forceinline__ float gate_mul(float g, float u, int kind, float limi
   return (g / (1.f + expf(-g))) * u;
 }
 
+// e^x in a few instructions (a result below the normal range may come out as 0, one above it as infinity): 2^t with
+// t = x log2(e) rounded, corrected by what the rounding of t lost, r = x log2(e) - t, as 2^t (1 + r ln 2); within two
+// units in the last place.
+__device__ __forceinline__ float short_exp(float x) {
+  const float L2E = 1.44269502162933349609375f, L2E_LO = 1.925963033500011e-8f;
+  const float t = x * L2E;
+  float r = fmaf(x, L2E, -t);
+  r = fmaf(x, L2E_LO, r);
+  const float e = __builtin_amdgcn_exp2f(t);
+  return fmaf(e, r * 0.693147182464599609375f, e);
+}
+
+// sigmoid(z) and z sigmoid(z) with that exponential and the hardware's reciprocal: within a few units in the last place
+// (the exponent is kept below the overflow: beyond 80 the results are e^z and z e^z, which is nothing, either way)
+__device__ __forceinline__ float short_sigmoid(float z) {
+  return __builtin_amdgcn_rcpf(1.f + short_exp(fminf(-z, 80.f)));
+}
+__device__ __forceinline__ float short_silu(float z) { return z * short_sigmoid(z); }
+
+// the first key that a query at position p sees: of its own run of `chunk` positions (counted from position 0) where
+// chunk > 0, of the last `window` keys where window > 0, else the first of all
+__device__ __forceinline__ int first_seen_key(int p, int window, int chunk) {
+  if (chunk > 0) return p - p % chunk;
+  return window > 0 ? max(0, p - window + 1) : 0;
+}
+
 // sin and cos of an angle of up to 4e6 rad (a position times a frequency of at most 1), to about
 // 1e-6: the library's sincosf spends over a thousand cycles on arguments this large.  The multiple
 // of 2 pi is taken off in three steps whose constants have few enough bits for the first two

@@ -69,13 +69,14 @@ extern "C" int sa_embed(const void* table, int table_dtype, const int* tokens, c
 
 // ---------------------------------------------------------------------------------------------
 // residual add + RMSNorm (serve/model.py:63-68,147-148):
-//   v = x[t] + delta[t];  x[t] = v (only when rows == nullptr);  y[r] = v * rsqrt(mean(v^2) + eps) * w
+//   v = x[t] + delta[t];  x[t] = v + after (only when rows == nullptr);  y[r] = v * rsqrt(mean(v^2) + eps) * w
+// after (fp32 [d], or null): a constant row that joins the stream behind the norm.
 // rows != nullptr: output row r takes source row rows[r] and x is left untouched.
 // ---------------------------------------------------------------------------------------------
 template <typename TA, typename TD, typename TW>
 __global__ void add_rmsnorm_kernel(float* __restrict__ x, const TD* __restrict__ delta, int parts,
                                    size_t part_stride, const TW* __restrict__ w, TA* __restrict__ y,
-                                   const int* __restrict__ rows, float eps, int d) {
+                                   const int* __restrict__ rows, const float* __restrict__ after, float eps, int d) {
   __shared__ float scratch[16];
   const int r = blockIdx.x;
   const int t = rows ? rows[r] : r;
@@ -97,6 +98,7 @@ __global__ void add_rmsnorm_kernel(float* __restrict__ x, const TD* __restrict__
     float v = xr[i];
     if (dr && rows)
       for (int p = 0; p < parts; ++p) v += to_float(dr[p * part_stride + i]);
+    if (after) xr[i] = v + after[i];              // (this thread's own element; with rows there is no `after`)
     yr[i] = from_float<TA>((v * rs) * to_float(w[i]));
   }
 }
@@ -124,7 +126,8 @@ template <typename TA, typename TD, typename TW, int PMAX>
 __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict__ x, const TD* __restrict__ delta,
                                                               int parts, size_t part_stride,
                                                               const TW* __restrict__ w, TA* __restrict__ y,
-                                                              const int* __restrict__ rows, float eps, int d) {
+                                                              const int* __restrict__ rows,
+                                                              const float* __restrict__ after, float eps, int d) {
   __shared__ float scratch[16];
   const int r = blockIdx.x;
   const int t = rows ? rows[r] : r;
@@ -163,7 +166,12 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict_
     const int gi = threadIdx.x + k * 256;
     const int i = gi * 4;
     if (k < nk && gi < groups) {
-      if (dr && !rows) store4(xr + i, v[k]);
+      if (after) {
+        const float4 c = load4(after + i);
+        store4(xr + i, make_float4(v[k].x + c.x, v[k].y + c.y, v[k].z + c.z, v[k].w + c.w));
+      } else if (dr && !rows) {
+        store4(xr + i, v[k]);
+      }
       store4(yr + i, make_float4((v[k].x * rs) * wv[k].x, (v[k].y * rs) * wv[k].y,
                                  (v[k].z * rs) * wv[k].z, (v[k].w * rs) * wv[k].w));
     }
@@ -173,10 +181,10 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict_
 // delta: [T, d] in the activation dtype (delta_dtype == act_dtype, parts == 1), or fp32
 // [parts, T, d] partial sums that are added in order.
 extern "C" int sa_add_rmsnorm(float* x, const void* delta, int delta_dtype, int parts, const void* w,
-                              int w_dtype, void* y, int act_dtype, const int* rows, float eps, int R,
-                              int T, int d, hipStream_t stream) {
+                              int w_dtype, void* y, int act_dtype, const int* rows, const float* after, float eps,
+                              int R, int T, int d, hipStream_t stream) {
   if (R <= 0) return 0;
-  if (d <= 0 || parts < 1) return SA_ERR_ARG;
+  if (d <= 0 || parts < 1 || (rows && after)) return SA_ERR_ARG;
   if (delta && delta_dtype != act_dtype && delta_dtype != SA_F32) return SA_ERR_UNSUPPORTED;
   if (delta && parts > 1 && delta_dtype != SA_F32) return SA_ERR_UNSUPPORTED;
   const size_t part_stride = (size_t)T * d;
@@ -186,16 +194,16 @@ extern "C" int sa_add_rmsnorm(float* x, const void* delta, int delta_dtype, int 
   do {                                                                                                   \
     if (vec && parts == 1)                                                                               \
       hipLaunchKernelGGL((add_rmsnorm_vec_kernel<TA, TD, TW, 1>), grid, block, 0, stream, x,             \
-                         (const TD*)delta, parts, part_stride, (const TW*)w, (TA*)y, rows, eps, d);      \
+                         (const TD*)delta, parts, part_stride, (const TW*)w, (TA*)y, rows, after, eps, d);      \
     else if (vec && parts <= 4)                                                                          \
       hipLaunchKernelGGL((add_rmsnorm_vec_kernel<TA, TD, TW, 4>), grid, block, 0, stream, x,             \
-                         (const TD*)delta, parts, part_stride, (const TW*)w, (TA*)y, rows, eps, d);      \
+                         (const TD*)delta, parts, part_stride, (const TW*)w, (TA*)y, rows, after, eps, d);      \
     else if (vec && parts <= 8)                                                                          \
       hipLaunchKernelGGL((add_rmsnorm_vec_kernel<TA, TD, TW, 8>), grid, block, 0, stream, x,             \
-                         (const TD*)delta, parts, part_stride, (const TW*)w, (TA*)y, rows, eps, d);      \
+                         (const TD*)delta, parts, part_stride, (const TW*)w, (TA*)y, rows, after, eps, d);      \
     else                                                                                                 \
       hipLaunchKernelGGL((add_rmsnorm_kernel<TA, TD, TW>), grid, block, 0, stream, x, (const TD*)delta,  \
-                         parts, part_stride, (const TW*)w, (TA*)y, rows, eps, d);                        \
+                         parts, part_stride, (const TW*)w, (TA*)y, rows, after, eps, d);                 \
   } while (0)
   const bool dfloat = delta && delta_dtype == SA_F32;
   if (act_dtype == SA_F32 && w_dtype == SA_F32) GO(float, float, float);

@@ -1,8 +1,12 @@
 // What lies between the q/k/v product and the attention of a mixer that norms its queries and keys:
 //
+//   q, k, v    += bias                                 (fp32, over the columns of a row; null: none)
+//   v[t, g, :] = k[t, g, :]                            (`shared`: the values are the keys as they are now)
 //   q[t, h, :] = N(q[t, h, :]) * wq * temp(p_t)       N(y) = y / sqrt(mean(y^2) + eps), per head,
 //   k[t, g, :] = N(k[t, g, :]) * wk                    one weight vector for all heads
 //   temp(p)    = 1 + coef * ln(floor((p + 1) / every) + 1)   (every <= 0: 1)
+//   q, k       <- the first `rot` dims of every head turned by the position: dim i pairs with i + rot / 2,
+//                 (u, v) -> (u cos a - v sin a, v cos a + u sin a), a = position * freq[i]     (rot 0: none)
 //   v[t, g, :] = (1 - lambda) v[t, g, :] + lambda v_first[t, g, :]   (v_first null: v as it is)
 //
 // then k and v of every token go to its cache slot and q into rows of its own.  Keys and queries have D
@@ -10,15 +14,24 @@
 // of 16): the places behind D (in q and k) and behind Dv (in v) are written as zeros, so that scores and
 // weighted sums are those of the unpadded heads.  All arithmetic is fp32, the template type is storage.
 //
-// Input rows are [Hq D | Hk D | Hk Dv] (one product); q_out [T, Hq Dp]; k pages [P, Hk, page_size, Dp],
+// Input rows are [Hq D | Hk D | Hk Dv] (one product; with `shared` no Hk Dv); q_out [T, Hq Dp]; k pages [P, Hk, page_size, Dp],
 // v pages [P, Hk, Dp, page_size]; slot[t] = page * page_size + offset, < 0: nothing stored.
 //
 // Two kernels: the general one (any sizes and alignments: a wave per (token, head), a lane an element at a time),
-// and one for sizes that are multiples of 8 from aligned rows, which moves 8 elements a lane (16 bytes of bf16):
+// and one for sizes that are multiples of 8 (rot of 16) from aligned rows, which moves 8 elements a lane (16 bytes of bf16):
 // its first blocks take the query and key heads, a group of lanes per head; its last blocks take the values with
 // neighbouring lanes on neighbouring tokens, so that the writes into the transposed value pages, where the
 // tokens of a page lie side by side, fall into common lines.
 #include "common.h"
+
+// sine and cosine of the float32 engine's angles are the library's, those of the bfloat16 engine's come from the
+// hardware's behind an argument reduction
+template <typename TA>
+__device__ __forceinline__ void rotation_of(float angle, float* sn, float* cs);
+template <>
+__device__ __forceinline__ void rotation_of<float>(float angle, float* sn, float* cs) { sincosf(angle, sn, cs); }
+template <>
+__device__ __forceinline__ void rotation_of<bf16_t>(float angle, float* sn, float* cs) { sincos_reduced(angle, sn, cs); }
 
 __device__ __forceinline__ float query_temp(const int* positions, int t, float coef, int every) {
   return every > 0 ? 1.f + coef * logf((float)((positions[t] + 1) / every) + 1.f) : 1.f;
@@ -29,7 +42,8 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_kernel(
     const TA* __restrict__ qkv, int row_stride, TA* __restrict__ q_out, const int* __restrict__ positions,
     const int* __restrict__ slot, TA* __restrict__ k_pages, TA* __restrict__ v_pages, const float* __restrict__ wq,
     const float* __restrict__ wk, float eps, float temp_coef, int temp_every, const TA* __restrict__ v_first,
-    int v_first_stride, float lambda, int Hq, int Hk, int D, int Dv, int Dp, int page_size) {
+    int v_first_stride, float lambda, const float* __restrict__ bias, const float* __restrict__ freq, int rot, int shared,
+    int Hq, int Hk, int D, int Dv, int Dp, int page_size) {
   const int t = blockIdx.x;
   const int lane = threadIdx.x & (SA_WAVE - 1);
   const int u = blockIdx.y * (blockDim.x / SA_WAVE) + threadIdx.x / SA_WAVE;      // the head this wave takes
@@ -45,9 +59,10 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_kernel(
     const int g = is_q ? u : u - Hq;
     if (!is_q && s < 0) return;
     const TA* x = row + (size_t)u * D;
+    const float* b = bias ? bias + (size_t)u * D : nullptr;
     float ss = 0.f;
     for (int i = lane; i < D; i += SA_WAVE) {
-      const float v = to_float(x[i]);
+      const float v = to_float(x[i]) + (b ? b[i] : 0.f);
       ss += v * v;
     }
     ss = wave_sum(ss);
@@ -55,10 +70,18 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_kernel(
     const float temp = is_q ? query_temp(positions, t, temp_coef, temp_every) : 1.f;
     const float* w = is_q ? wq : wk;
     TA* dst = is_q ? q_out + ((size_t)t * Hq + g) * Dp : k_pages + (((size_t)page * Hk + g) * page_size + off) * Dp;
+    const int half = rot >> 1;
     for (int i = lane; i < Dp; i += SA_WAVE) {
       TA o = zero;
       if (i < D) {
-        float v = (to_float(x[i]) * rs) * w[i];
+        float v = ((to_float(x[i]) + (b ? b[i] : 0.f)) * rs) * w[i];
+        if (i < rot) {
+          const int j = i < half ? i : i - half, ip = i < half ? i + half : i - half;
+          const float other = ((to_float(x[ip]) + (b ? b[ip] : 0.f)) * rs) * w[ip];
+          float sn, cs;
+          rotation_of<TA>((float)positions[t] * freq[j], &sn, &cs);
+          v = i < half ? v * cs - other * sn : v * cs + other * sn;
+        }
         if (is_q) v *= temp;
         o = from_float<TA>(v);
       }
@@ -68,13 +91,15 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_kernel(
   }
   if (s < 0) return;
   const int g = u - Hq - Hk;
-  const TA* x = row + (size_t)(Hq + Hk) * D + (size_t)g * Dv;
+  const size_t vcol = (size_t)(shared ? Hq : Hq + Hk) * D + (size_t)g * Dv;
+  const TA* x = row + vcol;
+  const float* b = bias ? bias + vcol : nullptr;
   const TA* f = v_first ? v_first + (size_t)t * v_first_stride + (size_t)g * Dv : nullptr;
   TA* dst = v_pages + ((size_t)page * Hk + g) * (size_t)Dp * page_size + off;
   for (int i = lane; i < Dp; i += SA_WAVE) {
     TA o = zero;
     if (i < Dv) {
-      float v = to_float(x[i]);
+      float v = to_float(x[i]) + (b ? b[i] : 0.f);
       if (f) v = (1.f - lambda) * v + lambda * to_float(f[i]);
       o = from_float<TA>(v);
     }
@@ -116,7 +141,8 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_vec_kernel(
     const TA* __restrict__ qkv, int row_stride, TA* __restrict__ q_out, const int* __restrict__ positions,
     const int* __restrict__ slot, TA* __restrict__ k_pages, TA* __restrict__ v_pages, const float* __restrict__ wq,
     const float* __restrict__ wk, float eps, float temp_coef, int temp_every, const TA* __restrict__ v_first,
-    int v_first_stride, float lambda, int T, int Hq, int Hk, int D, int Dv, int Dp, int page_size, int qk_blocks) {
+    int v_first_stride, float lambda, const float* __restrict__ bias, const float* __restrict__ freq, int rot, int shared,
+    int T, int Hq, int Hk, int D, int Dv, int Dp, int page_size, int qk_blocks) {
   if ((int)blockIdx.x < qk_blocks) {
     const int sub = threadIdx.x % LPH;
     const long long unit = (long long)blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
@@ -126,13 +152,20 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_vec_kernel(
     const bool is_q = u < Hq;
     const int i = sub * 8;
     float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (live && i < D) load8(qkv + (size_t)t * row_stride + (size_t)u * D + i, v);
+    if (live && i < D) {
+      load8(qkv + (size_t)t * row_stride + (size_t)u * D + i, v);
+      if (bias) {
+        float b[8];
+        load8(bias + (size_t)u * D + i, b);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) v[k] += b[k];
+      }
+    }
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < 8; ++k) ss += v[k] * v[k];
 #pragma unroll
     for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, SA_WAVE);
-    if (!live || i >= Dp) return;
     const float rs = 1.0f / sqrtf(ss / (float)D + eps);
     const float temp = is_q ? query_temp(positions, t, temp_coef, temp_every) : 1.f;
     if (i < D) {
@@ -144,6 +177,28 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_vec_kernel(
         if (is_q) v[k] *= temp;
       }
     }
+    if (rot > 0) {
+      // the other halves of this lane's eight pairs lie rot / 16 lanes away (every lane of the wave takes part)
+      const int hl = rot >> 4;
+      const bool first = sub < hl, turned = sub < 2 * hl;
+      const int base = (threadIdx.x & (SA_WAVE - 1)) - sub;
+      const int from = base + (turned ? (first ? sub + hl : sub - hl) : sub);
+      float other[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) other[k] = __shfl(v[k], from, SA_WAVE);
+      if (live && turned) {
+        float fr[8];
+        load8(freq + (first ? i : i - (rot >> 1)), fr);
+        const float pos = (float)positions[t];
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+          float sn, cs;
+          rotation_of<TA>(pos * fr[k], &sn, &cs);
+          v[k] = first ? v[k] * cs - other[k] * sn : v[k] * cs + other[k] * sn;
+        }
+      }
+    }
+    if (!live || i >= Dp) return;
     if (is_q) {
       store8(q_out + ((size_t)t * Hq + u) * Dp + i, v);
     } else {
@@ -166,7 +221,14 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_vec_kernel(
   const int page = s / page_size, off = s - page * page_size;
   float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
   if (i < Dv) {
-    load8(qkv + (size_t)t * row_stride + (size_t)(Hq + Hk) * D + (size_t)g * Dv + i, v);
+    const size_t vcol = (size_t)(shared ? Hq : Hq + Hk) * D + (size_t)g * Dv + i;
+    load8(qkv + (size_t)t * row_stride + vcol, v);
+    if (bias) {
+      float b[8];
+      load8(bias + vcol, b);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] += b[k];
+    }
     if (v_first) {
       float f[8];
       load8(v_first + (size_t)t * v_first_stride + (size_t)g * Dv + i, f);
@@ -182,11 +244,12 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_vec_kernel(
 template <typename TA>
 static int launch_qk_norm(const void* qkv, int row_stride, void* q_out, const int* positions, const int* slot,
                           void* k_pages, void* v_pages, const float* wq, const float* wk, float eps, float temp_coef,
-                          int temp_every, const void* v_first, int v_first_stride, float lambda, int T, int Hq, int Hk,
-                          int D, int Dv, int Dp, int page_size, hipStream_t stream) {
+                          int temp_every, const void* v_first, int v_first_stride, float lambda, const float* bias,
+                          const float* freq, int rot, int shared, int T, int Hq, int Hk, int D, int Dv, int Dp,
+                          int page_size, hipStream_t stream) {
   const uintptr_t bits = (uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)k_pages | (uintptr_t)v_pages |
-                         (uintptr_t)v_first | (uintptr_t)wq | (uintptr_t)wk;
-  const bool vec = ((D | Dv | Dp | row_stride | v_first_stride) & 7) == 0 && (bits & 15) == 0 && Dp <= 512;
+                         (uintptr_t)v_first | (uintptr_t)wq | (uintptr_t)wk | (uintptr_t)bias | (uintptr_t)freq;
+  const bool vec = ((D | Dv | Dp | row_stride | v_first_stride) & 7) == 0 && (rot & 15) == 0 && (bits & 15) == 0 && Dp <= 512;
   if (vec) {
     int lph = 2;
     while (lph * 8 < Dp) lph *= 2;
@@ -198,7 +261,8 @@ static int launch_qk_norm(const void* qkv, int row_stride, void* q_out, const in
 #define GOV(LPH)                                                                                                      \
   hipLaunchKernelGGL((qk_norm_kv_write_vec_kernel<TA, LPH>), grid, block, 0, stream, (const TA*)qkv, row_stride,       \
                      (TA*)q_out, positions, slot, (TA*)k_pages, (TA*)v_pages, wq, wk, eps, temp_coef, temp_every,     \
-                     (const TA*)v_first, v_first_stride, lambda, T, Hq, Hk, D, Dv, Dp, page_size, (int)qk_blocks)
+                     (const TA*)v_first, v_first_stride, lambda, bias, freq, rot, shared, T, Hq, Hk, D, Dv, Dp, page_size, \
+                     (int)qk_blocks)
     switch (lph) {
       case 2: GOV(2); break;
       case 4: GOV(4); break;
@@ -215,27 +279,30 @@ static int launch_qk_norm(const void* qkv, int row_stride, void* q_out, const in
   dim3 grid(T, (units + 3) / 4), block(256);
   hipLaunchKernelGGL(qk_norm_kv_write_kernel<TA>, grid, block, 0, stream, (const TA*)qkv, row_stride, (TA*)q_out,
                      positions, slot, (TA*)k_pages, (TA*)v_pages, wq, wk, eps, temp_coef, temp_every,
-                     (const TA*)v_first, v_first_stride, lambda, Hq, Hk, D, Dv, Dp, page_size);
+                     (const TA*)v_first, v_first_stride, lambda, bias, freq, rot, shared, Hq, Hk, D, Dv, Dp, page_size);
   return 0;
 }
 
 extern "C" int sa_qk_norm_kv_write(const void* qkv, int row_stride, void* q_out, int act_dtype, const int* positions,
                                    const int* slot, void* k_pages, void* v_pages, const float* wq, const float* wk,
                                    float eps, float temp_coef, int temp_every, const void* v_first, int v_first_stride,
-                                   float lambda, int T, int Hq, int Hk, int D, int Dv, int Dp, int page_size,
-                                   hipStream_t stream) {
+                                   float lambda, const float* bias, const float* freq, int rot, int shared, int T, int Hq,
+                                   int Hk, int D, int Dv, int Dp, int page_size, hipStream_t stream) {
   if (T <= 0) return 0;
   if (Hq <= 0 || Hk <= 0 || D <= 0 || Dv <= 0 || Dp < D || Dp < Dv || page_size <= 0 || !wq || !wk || !q_out)
     return SA_ERR_ARG;
-  if (row_stride < Hq * D + Hk * (D + Dv) || (slot && (!k_pages || !v_pages)) || (temp_every > 0 && !positions))
+  if (row_stride < Hq * D + Hk * (shared ? D : D + Dv) || (slot && (!k_pages || !v_pages)) ||
+      ((temp_every > 0 || rot > 0) && !positions) || (shared && D != Dv) || rot < 0 || rot % 2 || rot > D || (rot > 0 && !freq))
     return SA_ERR_ARG;
   int rc;
   if (act_dtype == SA_F32)
     rc = launch_qk_norm<float>(qkv, row_stride, q_out, positions, slot, k_pages, v_pages, wq, wk, eps, temp_coef,
-                               temp_every, v_first, v_first_stride, lambda, T, Hq, Hk, D, Dv, Dp, page_size, stream);
+                               temp_every, v_first, v_first_stride, lambda, bias, freq, rot, shared, T, Hq, Hk, D, Dv, Dp,
+                                page_size, stream);
   else if (act_dtype == SA_BF16)
     rc = launch_qk_norm<bf16_t>(qkv, row_stride, q_out, positions, slot, k_pages, v_pages, wq, wk, eps, temp_coef,
-                                temp_every, v_first, v_first_stride, lambda, T, Hq, Hk, D, Dv, Dp, page_size, stream);
+                                temp_every, v_first, v_first_stride, lambda, bias, freq, rot, shared, T, Hq, Hk, D, Dv, Dp,
+                                page_size, stream);
   else
     return SA_ERR_UNSUPPORTED;
   if (rc != 0) return rc;

@@ -15,20 +15,6 @@
 
 #define RS_MAX_TAPS 16
 
-// e^x in a few instructions (a result below the normal range may come out as 0, one above it as infinity): 2^t with t = x log2(e) rounded, corrected by what the rounding of t lost, r = x log2(e) - t, as
-// 2^t (1 + r ln 2).  A few instructions, and within two units in the last place.
-__device__ __forceinline__ float rs_exp(float x) {
-  const float L2E = 1.44269502162933349609375f, L2E_LO = 1.925963033500011e-8f;
-  const float t = x * L2E;
-  float r = fmaf(x, L2E, -t);
-  r = fmaf(x, L2E_LO, r);
-  const float e = __builtin_amdgcn_exp2f(t);
-  return fmaf(e, r * 0.693147182464599609375f, e);
-}
-
-// z sigmoid(z) with that exponential and the hardware's reciprocal: within a few units in the last place
-// (the exponent is kept below the overflow: beyond 80 the result is z e^z, which is nothing, either way)
-__device__ __forceinline__ float rs_silu(float z) { return z * __builtin_amdgcn_rcpf(1.f + rs_exp(fminf(-z, 80.f))); }
 __device__ __forceinline__ float rs_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 // ln(sigmoid(z)) without overflow on either side
 __device__ __forceinline__ float rs_logsigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
@@ -46,6 +32,13 @@ __device__ __forceinline__ float row16_sum(float v) {
   return v;
 }
 
+// a projected value as it enters the recurrence: as it is, or behind z sigmoid(z)
+template <typename T>
+__device__ __forceinline__ float read_qkv(T x, int silu) {
+  const float z = to_float(x);
+  return silu ? short_silu(z) : z;
+}
+
 // ---------------------------------------------------------------------------------------------
 // The recurrence.  grid (column tiles, H, B), 256 threads = 16 groups of columns x 16 parts of the rows: thread
 // (cl, r) keeps rows r RPT .. r RPT + RPT - 1 of columns (tile 16 + cl) CPT .. + CPT - 1 in registers for the whole
@@ -60,7 +53,8 @@ __device__ __forceinline__ float row16_sum(float v) {
 template <typename TQ, int RPT, int CPT, int CH>
 __global__ __launch_bounds__(256) void decay_scan_kernel(
     const TQ* __restrict__ q, const TQ* __restrict__ k, const TQ* __restrict__ v, long long q_stride,
-    long long k_stride, long long v_stride, const float* __restrict__ log_decay, int per_channel, float q_scale,
+    long long k_stride, long long v_stride, const float* __restrict__ log_decay, int per_channel,
+    long long decay_stride, int silu, float q_scale,
     float* __restrict__ state, long long state_stride, const int* __restrict__ cu_q,
     const int* __restrict__ state_slots, float* __restrict__ o, int H, int Hk, int dk, int dv) {
   constexpr int ROWS = 16 * RPT;
@@ -93,9 +87,9 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(
       const bool in = i < dk;
       const size_t tok = (size_t)(t0 + c0 + tt);
       const int ic = in ? i : 0;
-      const float qv = to_float(q[tok * q_stride + (size_t)hk * dk + ic]) * q_scale;
-      const float kv = to_float(k[tok * k_stride + (size_t)hk * dk + ic]);
-      const float av = expf(per_channel ? log_decay[(tok * H + h) * (size_t)dk + ic] : log_decay[tok * H + h]);
+      const float qv = read_qkv(q[tok * q_stride + (size_t)hk * dk + ic], silu) * q_scale;
+      const float kv = read_qkv(k[tok * k_stride + (size_t)hk * dk + ic], silu);
+      const float av = expf(log_decay[tok * decay_stride + (per_channel ? (size_t)h * dk + ic : (size_t)h)]);
       sq[tt][pos] = in ? qv : 0.f;
       sk[tt][pos] = in ? kv : 0.f;
       sa[tt][pos] = in ? av : 1.f;
@@ -103,7 +97,7 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(
     for (int idx = threadIdx.x; idx < m * 16 * CPT; idx += 256) {
       const int tt = idx / (16 * CPT), c = idx - tt * (16 * CPT);
       const int jj = tile * 16 * CPT + c;
-      sv[tt][c] = jj < dv ? to_float(v[(size_t)(t0 + c0 + tt) * v_stride + (size_t)h * dv + jj]) : 0.f;
+      sv[tt][c] = jj < dv ? read_qkv(v[(size_t)(t0 + c0 + tt) * v_stride + (size_t)h * dv + jj], silu) : 0.f;
     }
     __syncthreads();
     for (int tt = 0; tt < m; ++tt) {
@@ -157,23 +151,23 @@ extern "C" long long sa_decay_scan_state_floats(int H, int dk, int dv) {
 
 template <typename TQ, int RPT, int CPT>
 static void launch_scan(const void* q, const void* k, const void* v, long long qs, long long ks, long long vs,
-                        const float* decay, int per_channel, float q_scale, float* state, long long state_stride,
+                        const float* decay, int per_channel, long long decay_stride, int silu, float q_scale, float* state, long long state_stride,
                         const int* cu_q, const int* slots, float* o, int B, int H, int Hk, int dk, int dv,
                         hipStream_t stream) {
   constexpr int CH = RPT >= 16 ? 8 : 16;
   const int tiles = (dv + 16 * CPT - 1) / (16 * CPT);
   dim3 grid(tiles, H, B), block(256);
   hipLaunchKernelGGL((decay_scan_kernel<TQ, RPT, CPT, CH>), grid, block, 0, stream, (const TQ*)q, (const TQ*)k,
-                     (const TQ*)v, qs, ks, vs, decay, per_channel, q_scale, state, state_stride, cu_q, slots, o, H, Hk,
+                     (const TQ*)v, qs, ks, vs, decay, per_channel, decay_stride, silu, q_scale, state, state_stride, cu_q, slots, o, H, Hk,
                      dk, dv);
 }
 
 template <typename TQ, int RPT>
 static void launch_scan_c(int cpt, const void* q, const void* k, const void* v, long long qs, long long ks,
-                          long long vs, const float* decay, int per_channel, float q_scale, float* state,
+                          long long vs, const float* decay, int per_channel, long long decay_stride, int silu, float q_scale, float* state,
                           long long state_stride, const int* cu_q, const int* slots, float* o, int B, int H, int Hk,
                           int dk, int dv, hipStream_t stream) {
-#define GO(C) launch_scan<TQ, RPT, C>(q, k, v, qs, ks, vs, decay, per_channel, q_scale, state, state_stride, cu_q, slots, o, B, H, Hk, dk, dv, stream)
+#define GO(C) launch_scan<TQ, RPT, C>(q, k, v, qs, ks, vs, decay, per_channel, decay_stride, silu, q_scale, state, state_stride, cu_q, slots, o, B, H, Hk, dk, dv, stream)
   if (cpt == 4) GO(4);
   else if (cpt == 2) GO(2);
   else GO(1);
@@ -182,10 +176,10 @@ static void launch_scan_c(int cpt, const void* q, const void* k, const void* v, 
 
 template <typename TQ>
 static void launch_scan_r(int rpt, int cpt, const void* q, const void* k, const void* v, long long qs, long long ks,
-                          long long vs, const float* decay, int per_channel, float q_scale, float* state,
+                          long long vs, const float* decay, int per_channel, long long decay_stride, int silu, float q_scale, float* state,
                           long long state_stride, const int* cu_q, const int* slots, float* o, int B, int H, int Hk,
                           int dk, int dv, hipStream_t stream) {
-#define GO(R) launch_scan_c<TQ, R>(cpt, q, k, v, qs, ks, vs, decay, per_channel, q_scale, state, state_stride, cu_q, slots, o, B, H, Hk, dk, dv, stream)
+#define GO(R) launch_scan_c<TQ, R>(cpt, q, k, v, qs, ks, vs, decay, per_channel, decay_stride, silu, q_scale, state, state_stride, cu_q, slots, o, B, H, Hk, dk, dv, stream)
   switch (rpt) {
     case 1: GO(1); break;
     case 2: GO(2); break;
@@ -227,7 +221,8 @@ enum { RS_WHOLE = 0, RS_PIECE_STATES = 1, RS_PIECE_OUTPUTS = 2 };
 template <typename TQ, int NT>
 __global__ __launch_bounds__(256) void decay_scan_block_kernel(
     const TQ* __restrict__ q, const TQ* __restrict__ k, const TQ* __restrict__ v, long long q_stride,
-    long long k_stride, long long v_stride, const float* __restrict__ log_decay, int per_channel, float q_scale,
+    long long k_stride, long long v_stride, const float* __restrict__ log_decay, int per_channel,
+    long long decay_stride, int silu, float q_scale,
     float* __restrict__ state, long long state_stride, const int* __restrict__ cu_q,
     const int* __restrict__ state_slots, float* __restrict__ o, int H, int Hk, int dk, int dv, int RPT, int CPT,
     int mode, int piece, int pieces, float* __restrict__ scratch, long long scratch_stride, long long scratch_decays) {
@@ -285,7 +280,7 @@ __global__ __launch_bounds__(256) void decay_scan_block_kernel(
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
       const unsigned tt = (unsigned)min(t, last);
-      lo[t] = per_channel ? (tt * H) * (unsigned)dk + c : tt * H;
+      lo[t] = tt * (unsigned)decay_stride + (per_channel ? c : 0u);
     }
 #pragma unroll
     for (int e = 0; e < NE; ++e) {
@@ -300,7 +295,7 @@ __global__ __launch_bounds__(256) void decay_scan_block_kernel(
   };
   auto fetch = [&](int c0) {
     const size_t tok = (size_t)(t0 + c0);
-    const float* lb = log_decay + (per_channel ? (tok * H + h) * (size_t)dk : tok * H + h);
+    const float* lb = log_decay + tok * decay_stride + (per_channel ? (size_t)h * dk : (size_t)h);
     const TQ* qb = q + tok * q_stride + (size_t)hk * dk;
     const TQ* kb = k + tok * k_stride + (size_t)hk * dk;
     const TQ* vb = v + tok * v_stride + (size_t)h * dv;
@@ -330,27 +325,27 @@ __global__ __launch_bounds__(256) void decay_scan_block_kernel(
         sb[t][tid] = run;
         if (t == 7) b7 = run;
       }
-      sdec[tid] = rs_exp(run);
+      sdec[tid] = short_exp(run);
       btotal += run;
       far = (b7 < -RS_RANGE) || (run - b7 < -RS_RANGE);
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int idx = tid + 256 * e;
-      sv[idx >> 6][idx & 63] = ((idx >> 6) < m && tile * 64 + (idx & 63) < dv) ? to_float(rv[e]) : 0.f;
+      sv[idx >> 6][idx & 63] = ((idx >> 6) < m && tile * 64 + (idx & 63) < dv) ? read_qkv(rv[e], silu) : 0.f;
     }
     const int wide = __syncthreads_or(far);
 #pragma unroll
     for (int e = 0; e < NE; ++e) {
       const int idx = tid + 256 * e, t = idx / DKP, c = idx % DKP;
       const bool in = t < m && c < dk;
-      const float qv = in ? to_float(rq[e]) * q_scale : 0.f, kv = in ? to_float(rk[e]) : 0.f;
+      const float qv = in ? read_qkv(rq[e], silu) * q_scale : 0.f, kv = in ? read_qkv(rk[e], silu) : 0.f;
       const float bt = sb[t][c], b7 = sb[7][c], b15 = sb[15][c];
-      skt[t][c] = kv * rs_exp(b15 - bt);
+      skt[t][c] = kv * short_exp(b15 - bt);
       if (mode != RS_PIECE_STATES) {
-        sqh[t][c] = qv * rs_exp(bt);
-        sqp[t][c] = wide ? qv : qv * rs_exp(bt - b7);
-        skp[t][c] = wide ? kv : kv * rs_exp(b7 - bt);
+        sqh[t][c] = qv * short_exp(bt);
+        sqp[t][c] = wide ? qv : qv * short_exp(bt - b7);
+        skp[t][c] = wide ? kv : kv * short_exp(b7 - bt);
       }
     }
     if (c0 + 16 < n) {                           // in flight while the products run
@@ -375,7 +370,7 @@ __global__ __launch_bounds__(256) void decay_scan_block_kernel(
       const int t = tid >> 4, s = tid & 15;
       float a = 0.f;
       if (s <= t)
-        for (int c = 0; c < DKP; ++c) a = fmaf(sqp[t][c] * skp[s][c], rs_exp(sb[t][c] - sb[s][c]), a);
+        for (int c = 0; c < DKP; ++c) a = fmaf(sqp[t][c] * skp[s][c], short_exp(sb[t][c] - sb[s][c]), a);
       sam[t][s] = a;
     }
     __syncthreads();
@@ -419,7 +414,7 @@ __global__ __launch_bounds__(256) void decay_scan_block_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) st[state_at(16 * m + 4 * g + r)] = S[m][r];
   }
-  if (mode == RS_PIECE_STATES && tile == 0 && tid < DKP) mine[scratch_decays + (size_t)h * DKP + tid] = rs_exp(btotal);
+  if (mode == RS_PIECE_STATES && tile == 0 && tid < DKP) mine[scratch_decays + (size_t)h * DKP + tid] = short_exp(btotal);
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -458,12 +453,12 @@ __global__ __launch_bounds__(256) void decay_scan_chain_kernel(float* __restrict
 
 template <typename TQ>
 static int launch_scan_block(int rpt, int cpt, const void* q, const void* k, const void* v, long long qs, long long ks,
-                             long long vs, const float* decay, int per_channel, float q_scale, float* state,
+                             long long vs, const float* decay, int per_channel, long long decay_stride, int silu, float q_scale, float* state,
                              long long state_stride, const int* cu_q, const int* slots, float* o, int B, int H, int Hk,
                              int dk, int dv, int mode, int piece, int pieces, float* scratch, long long scratch_stride,
                              long long scratch_decays, hipStream_t stream) {
   dim3 grid((dv + 63) / 64, H, B * pieces), block(256);
-#define GO(N) hipLaunchKernelGGL((decay_scan_block_kernel<TQ, N>), grid, block, 0, stream, (const TQ*)q, (const TQ*)k, (const TQ*)v, qs, ks, vs, decay, per_channel, q_scale, state, state_stride, cu_q, slots, o, H, Hk, dk, dv, rpt, cpt, mode, piece, pieces, scratch, scratch_stride, scratch_decays)
+#define GO(N) hipLaunchKernelGGL((decay_scan_block_kernel<TQ, N>), grid, block, 0, stream, (const TQ*)q, (const TQ*)k, (const TQ*)v, qs, ks, vs, decay, per_channel, decay_stride, silu, q_scale, state, state_stride, cu_q, slots, o, H, Hk, dk, dv, rpt, cpt, mode, piece, pieces, scratch, scratch_stride, scratch_decays)
   switch (rpt) {
     case 1: GO(1); break;
     case 2: GO(2); break;
@@ -482,12 +477,13 @@ extern "C" int sa_decay_scan_block_min_tokens() { return RS_BLOCK_MIN_TOKENS; }
 
 // q, k: rows of `q_stride` / `k_stride` elements with head hk's dk values at hk dk (Hk heads; head h reads hk = h / (H / Hk));
 // v: rows of `v_stride` with head h's dv values at h dv; decay: the decays' logarithms, fp32 [T, H, dk] (per_channel) or [T, H];
+// (decay_stride floats from one token's to the next's; 0: the same for every token); silu: q, k and v pass z sigmoid(z);
 // o fp32 [T, H, dv]; max_q: the longest segment (what decides between the two kernels);
 // state: a request's row at state + slot state_stride (the floats that sa_decay_scan_state_floats counts), slot < 0: a
 // segment without a request, which starts from zeros and keeps nothing.
 extern "C" int sa_decay_scan(const void* q, const void* k, const void* v, int dtype, long long q_stride,
                              long long k_stride, long long v_stride, const float* decay, int per_channel,
-                             float q_scale, float* state, long long state_stride, const int* cu_q,
+                             long long decay_stride, int silu, float q_scale, float* state, long long state_stride, const int* cu_q,
                              const int* state_slots, float* o, int B, int H, int Hk, int dk, int dv, int max_q,
                              int piece, float* scratch, long long scratch_stride, hipStream_t stream) {
   if (B <= 0) return 0;
@@ -512,10 +508,10 @@ extern "C" int sa_decay_scan(const void* q, const void* k, const void* v, int dt
     const int modes[2] = {pieces > 1 ? RS_PIECE_STATES : RS_WHOLE, RS_PIECE_OUTPUTS};
     for (int pass = 0; pass < (pieces > 1 ? 2 : 1); ++pass) {
       const int rc = dtype == SA_F32
-          ? launch_scan_block<float>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, q_scale, state,
+          ? launch_scan_block<float>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, decay_stride, silu, q_scale, state,
                                      state_stride, cu_q, state_slots, o, B, H, Hk, dk, dv, modes[pass], piece, pieces,
                                      scratch, scratch_stride, floats, stream)
-          : launch_scan_block<bf16_t>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, q_scale, state,
+          : launch_scan_block<bf16_t>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, decay_stride, silu, q_scale, state,
                                       state_stride, cu_q, state_slots, o, B, H, Hk, dk, dv, modes[pass], piece, pieces,
                                       scratch, scratch_stride, floats, stream);
       if (rc) return rc;
@@ -531,10 +527,10 @@ extern "C" int sa_decay_scan(const void* q, const void* k, const void* v, int dt
     return 0;
   }
   if (dtype == SA_F32)
-    launch_scan_r<float>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, q_scale, state,
+    launch_scan_r<float>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, decay_stride, silu, q_scale, state,
                          state_stride, cu_q, state_slots, o, B, H, Hk, dk, dv, stream);
   else if (dtype == SA_BF16)
-    launch_scan_r<bf16_t>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, q_scale, state,
+    launch_scan_r<bf16_t>(rpt, cpt, q, k, v, q_stride, k_stride, v_stride, decay, per_channel, decay_stride, silu, q_scale, state,
                           state_stride, cu_q, state_slots, o, B, H, Hk, dk, dv, stream);
   else
     return SA_ERR_UNSUPPORTED;
@@ -619,7 +615,7 @@ __global__ __launch_bounds__(256) void ssm_prepare_kernel(
 #pragma unroll
         for (int j = 0; j < RS_MAX_TAPS; ++j)
           if (j < taps) acc = fmaf(w[j], xin[tt + j], acc);
-        const float y = rs_silu(acc);
+        const float y = short_silu(acc);
         const int t = t_first + tt;
         xbc[(size_t)t * C + c] = y;
         if (c < H * P) vout[(size_t)t * H * P + c] = sdt[tt][c / P - h_first] * y;
@@ -646,7 +642,7 @@ __global__ __launch_bounds__(256) void ssm_prepare_kernel(
       else xv = cs ? cs[(size_t)(taps - 1 + tp - t0) * C + c] : 0.f;
       acc = fmaf(conv_w[(size_t)c * taps + j], xv, acc);
     }
-    const float y = rs_silu(acc);
+    const float y = short_silu(acc);
     xbc[(size_t)t * C + c] = y;
     if (c < H * P) vout[(size_t)t * H * P + c] = sdt[t - blockIdx.x * per][c / P - h_first] * y;
   }
@@ -729,8 +725,13 @@ extern "C" int sa_conv_state_update(const void* zx, int dtype, long long zs, int
 //   u = o + skip_d[h] skip_x[t, i]                 (skip_x null: u = o)
 //   gate_first:  u <- u silu(g[t, i]);  y = u / sqrt(mean_group(u^2) + eps) * w[i % wn]
 //   else:        y = u / sqrt(mean_group(u^2) + eps) * w[i % wn] * silu(g[t, i])
-// g: rows of gate_stride elements in the output's storage type, read from column gate_col on.
+// (gate_kind 1: sigmoid(g) in place of silu(g)).  g: rows of gate_stride elements in the output's storage type, read from column gate_col on.
 // ---------------------------------------------------------------------------------------------
+__device__ __forceinline__ float readout_gate(float z, int kind) {
+  const float s = short_sigmoid(z);
+  return kind == 1 ? s : z * s;
+}
+
 // WAVES: how many waves share a group (1: a wave a group, four groups a workgroup of 256; 16: a workgroup of 1024 a
 // group, for groups of thousands, where a few waves' chains of loads and divisions would decide the time of a
 // decode step)
@@ -738,8 +739,8 @@ template <typename TA, int WAVES>
 __global__ __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) void gated_group_norm_kernel(
     const float* __restrict__ o, const float* __restrict__ skip_x, long long skip_stride,
     const float* __restrict__ skip_d, int dv, const TA* __restrict__ gate, long long gate_stride, int gate_col,
-    const float* __restrict__ w, int wn, int group, int gate_first, float eps, TA* __restrict__ y, long long units,
-    int n) {
+    const float* __restrict__ w, int wn, int group, int gate_first, int gate_kind, float eps, TA* __restrict__ y,
+    long long units, int n) {
   __shared__ float part[WAVES];
   constexpr int LANES = SA_WAVE * WAVES;
   const int lane = threadIdx.x & (LANES - 1);
@@ -773,7 +774,7 @@ __global__ __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) void gated_group_nor
       const int e = lane + x * LANES, i = i0 + min(e, group - 1);
       float u = ro[x];
       if (skip_x) u = fmaf(skip_d[i / dv], rx[x], u);
-      const float g = rs_silu(to_float(rg[x]));
+      const float g = readout_gate(to_float(rg[x]), gate_kind);
       if (gate_first) u *= g;
       if (e >= group) u = 0.f;
       ku[x] = u;
@@ -785,7 +786,7 @@ __global__ __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) void gated_group_nor
       const int i = i0 + e;
       float u = orow[i];
       if (skip_x) u = fmaf(skip_d[i / dv], skip_x[(size_t)t * skip_stride + i], u);
-      if (gate_first) u *= rs_silu(to_float(grow[i]));
+      if (gate_first) u *= readout_gate(to_float(grow[i]), gate_kind);
       ss = fmaf(u, u, ss);
     }
   }
@@ -815,7 +816,7 @@ __global__ __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) void gated_group_nor
     const int i = i0 + e;
     float u = orow[i];
     if (skip_x) u = fmaf(skip_d[i / dv], skip_x[(size_t)t * skip_stride + i], u);
-    const float g = rs_silu(to_float(grow[i]));
+    const float g = readout_gate(to_float(grow[i]), gate_kind);
     if (gate_first) u *= g;
     float out = (u * rs) * w[i % wn];
     if (!gate_first) out *= g;
@@ -825,17 +826,18 @@ __global__ __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) void gated_group_nor
 
 extern "C" int sa_gated_group_norm(const float* o, const float* skip_x, long long skip_stride, const float* skip_d,
                                    int dv, const void* gate, int dtype, long long gate_stride, int gate_col,
-                                   const float* w, int wn, int group, int gate_first, float eps, void* y, int T, int n,
+                                   const float* w, int wn, int group, int gate_first, int gate_kind, float eps, void* y, int T, int n,
                                    hipStream_t stream) {
   if (T <= 0) return 0;
-  if (!o || !gate || !w || !y || n <= 0 || group <= 0 || n % group || wn <= 0 || dv <= 0 || (skip_x && !skip_d))
+  if (!o || !gate || !w || !y || n <= 0 || group <= 0 || n % group || wn <= 0 || dv <= 0 || (skip_x && !skip_d) || gate_kind < 0 ||
+      gate_kind > 1)
     return SA_ERR_ARG;
   const long long units = (long long)T * (n / group);
   const bool whole = group >= 1024;             // a workgroup a group
   const long long blocks = whole ? units : (units + 3) / 4;
   if (blocks > 0x7fffffffLL) return SA_ERR_ARG;
   dim3 grid((unsigned)blocks), block(whole ? 1024 : 256);
-#define GO(TA, W) hipLaunchKernelGGL((gated_group_norm_kernel<TA, W>), grid, block, 0, stream, o, skip_x, skip_stride, skip_d, dv, (const TA*)gate, gate_stride, gate_col, w, wn, group, gate_first, eps, (TA*)y, units, n)
+#define GO(TA, W) hipLaunchKernelGGL((gated_group_norm_kernel<TA, W>), grid, block, 0, stream, o, skip_x, skip_stride, skip_d, dv, (const TA*)gate, gate_stride, gate_col, w, wn, group, gate_first, gate_kind, eps, (TA*)y, units, n)
   if (dtype == SA_F32) {
     if (whole) GO(float, 16); else GO(float, 1);
   } else if (dtype == SA_BF16) {

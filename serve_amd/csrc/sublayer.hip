@@ -1,4 +1,4 @@
-// Elementwise kernels of layers whose norm sits on the sublayer's output:
+// Elementwise and row kernels of layers whose norm sits on the sublayer's output:
 //   x <- x + s * N(y),  N(y) = y / sqrt(mean(y^2) + eps) * w      (x: fp32 residual stream)
 // and of feed-forwards with a plain activation between two products.  fp32 arithmetic; the
 // storage types of activations are templated.
@@ -332,6 +332,193 @@ extern "C" int sa_sigmoid_mul(void* a, const void* g, int act_dtype, long long n
   else if (act_dtype == SA_BF16)
     hipLaunchKernelGGL(sigmoid_mul_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)a, (const bf16_t*)g, (size_t)n);
   else return SA_ERR_UNSUPPORTED;
+  SA_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------------------------------------
+// A polynomial of normed powers as a feed-forward's activation, per row z of n values:
+//   y = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3,   powers element by element, N(v) = v / sqrt(mean(v^2) + eps)
+// Given the row's sums of z^2, z^4 and z^6 this is a polynomial in z with three row scalars.  z: [T, n] in the storage
+// type TZ, or fp32 [parts, T, n] partial sums that are added in order.  One workgroup a row; a thread keeps NG groups of
+// four values (TPB threads) between the two passes, as many as the row needs; rows that are longer, or that are no
+// multiple of four, go an element at a time and are read twice.
+// ---------------------------------------------------------------------------------------------
+struct PowerScales {
+  float r1, r2, r3;
+};
+
+// block sums of the three powers' squares -> the factors of z, z^2 and z^3
+__device__ __forceinline__ PowerScales power_scales(float s2, float s4, float s6, const float* __restrict__ coef, int n,
+                                                    float eps, float* part) {
+  const int lane = threadIdx.x & (SA_WAVE - 1), wave = threadIdx.x / SA_WAVE, waves = blockDim.x / SA_WAVE;
+  s2 = wave_sum(s2);
+  s4 = wave_sum(s4);
+  s6 = wave_sum(s6);
+  if (lane == 0) {
+    part[3 * wave] = s2;
+    part[3 * wave + 1] = s4;
+    part[3 * wave + 2] = s6;
+  }
+  __syncthreads();
+  s2 = s4 = s6 = 0.f;
+  for (int w = 0; w < waves; ++w) {
+    s2 += part[3 * w];
+    s4 += part[3 * w + 1];
+    s6 += part[3 * w + 2];
+  }
+  PowerScales p;
+  p.r1 = coef[0] / sqrtf(s2 / (float)n + eps);
+  p.r2 = coef[1] / sqrtf(s4 / (float)n + eps);
+  p.r3 = coef[2] / sqrtf(s6 / (float)n + eps);
+  return p;
+}
+
+__device__ __forceinline__ float power_sum(float z, const PowerScales& p, float c) {
+  return fmaf(fmaf(fmaf(p.r3, z, p.r2), z, p.r1), z, c);
+}
+
+template <typename TZ, typename TA, int NG, int PMAX>
+__global__ __launch_bounds__(1024) void poly_norm_vec_kernel(const TZ* __restrict__ z, int parts, size_t part_stride,
+                                                             const float* __restrict__ coef, float eps,
+                                                             TA* __restrict__ y, int n) {
+  __shared__ float part[48];
+  const TZ* row = z + (size_t)blockIdx.x * n;
+  const int groups = n >> 2, bd = blockDim.x;
+  float4 v[NG];
+#pragma unroll
+  for (int k = 0; k < NG; ++k) {
+    const int i = min((int)threadIdx.x + k * bd, groups - 1) * 4;
+    v[k] = ld4(row + i);
+    if (PMAX > 1) {
+#pragma unroll
+      for (int q = 1; q < PMAX; ++q) {
+        const float4 a = ld4(row + (size_t)min(q, parts - 1) * part_stride + i);
+        const float on = q < parts ? 1.f : 0.f;
+        v[k].x += on * a.x; v[k].y += on * a.y; v[k].z += on * a.z; v[k].w += on * a.w;
+      }
+    }
+  }
+  float s2 = 0.f, s4 = 0.f, s6 = 0.f;
+#pragma unroll
+  for (int k = 0; k < NG; ++k) {
+    const float in = (int)threadIdx.x + k * bd < groups ? 1.f : 0.f;
+    const float e[4] = {v[k].x, v[k].y, v[k].z, v[k].w};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float a = in * e[j] * e[j];
+      s2 += a;
+      s4 = fmaf(a, a, s4);
+      s6 = fmaf(a * a, a, s6);
+    }
+  }
+  const PowerScales p = power_scales(s2, s4, s6, coef, n, eps, part);
+  const float c = coef[3];
+  TA* out = y + (size_t)blockIdx.x * n;
+#pragma unroll
+  for (int k = 0; k < NG; ++k) {
+    const int gi = threadIdx.x + k * bd;
+    if (gi < groups)
+      st4(out + gi * 4, make_float4(power_sum(v[k].x, p, c), power_sum(v[k].y, p, c), power_sum(v[k].z, p, c),
+                                    power_sum(v[k].w, p, c)));
+  }
+}
+
+template <typename TZ, typename TA>
+__global__ __launch_bounds__(1024) void poly_norm_kernel(const TZ* __restrict__ z, int parts, size_t part_stride,
+                                                         const float* __restrict__ coef, float eps, TA* __restrict__ y,
+                                                         int n) {
+  __shared__ float part[48];
+  const TZ* row = z + (size_t)blockIdx.x * n;
+  float s2 = 0.f, s4 = 0.f, s6 = 0.f;
+  for (int i = threadIdx.x; i < n; i += blockDim.x) {
+    float v = 0.f;
+    for (int q = 0; q < parts; ++q) v += to_float(row[q * part_stride + i]);
+    const float a = v * v;
+    s2 += a;
+    s4 = fmaf(a, a, s4);
+    s6 = fmaf(a * a, a, s6);
+  }
+  const PowerScales p = power_scales(s2, s4, s6, coef, n, eps, part);
+  const float c = coef[3];
+  for (int i = threadIdx.x; i < n; i += blockDim.x) {
+    float v = 0.f;
+    for (int q = 0; q < parts; ++q) v += to_float(row[q * part_stride + i]);
+    y[(size_t)blockIdx.x * n + i] = from_float<TA>(power_sum(v, p, c));
+  }
+}
+
+template <typename TZ, typename TA>
+static void launch_poly_norm(const void* z, int parts, const float* coef, float eps, void* y, int T, int n,
+                             hipStream_t stream) {
+  const size_t part_stride = (size_t)T * n;
+  const int groups = n / 4;
+  // few rows: more threads a row (a row is a chain of a load, two sums and a store)
+  const int threads = groups <= 64 ? 64 : (groups <= 256 ? 256 : (T <= 256 || groups > 2048 ? 1024 : 256));
+  const int ng = (groups + threads - 1) / threads;
+  const bool vec = (n & 3) == 0 && (((uintptr_t)z | (uintptr_t)y) & 15) == 0 && ng <= 8 && parts <= 8;
+#define GO(NG, PM)                                                                                              \
+  hipLaunchKernelGGL((poly_norm_vec_kernel<TZ, TA, NG, PM>), dim3(T), dim3(threads), 0, stream, (const TZ*)z, parts, \
+                     part_stride, coef, eps, (TA*)y, n)
+#define GON(PM)               \
+  do {                        \
+    if (ng <= 1) GO(1, PM);   \
+    else if (ng <= 2) GO(2, PM); \
+    else if (ng <= 4) GO(4, PM); \
+    else GO(8, PM);           \
+  } while (0)
+  if (vec && parts == 1) GON(1);
+  else if (vec && parts <= 4) GON(4);
+  else if (vec) GON(8);
+  else
+    hipLaunchKernelGGL((poly_norm_kernel<TZ, TA>), dim3(T), dim3(n >= 1024 ? 1024 : 256), 0, stream, (const TZ*)z, parts,
+                       part_stride, coef, eps, (TA*)y, n);
+#undef GON
+#undef GO
+}
+
+extern "C" int sa_poly_norm(const void* z, int z_dtype, int parts, const float* coef, float eps, void* y, int y_dtype, int T,
+                            int n, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (!z || !coef || !y || n <= 0 || parts < 1) return SA_ERR_ARG;
+  if (parts > 1 && z_dtype != SA_F32) return SA_ERR_UNSUPPORTED;
+  if (z_dtype == SA_F32 && y_dtype == SA_F32) launch_poly_norm<float, float>(z, parts, coef, eps, y, T, n, stream);
+  else if (z_dtype == SA_F32 && y_dtype == SA_BF16) launch_poly_norm<float, bf16_t>(z, parts, coef, eps, y, T, n, stream);
+  else if (z_dtype == SA_BF16 && y_dtype == SA_BF16) launch_poly_norm<bf16_t, bf16_t>(z, parts, coef, eps, y, T, n, stream);
+  else return SA_ERR_UNSUPPORTED;
+  SA_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------------------------------------
+// y = cap tanh(scale y / cap) in place (cap 0: y = scale y): an output matrix's values, scaled and kept within a cap
+// ---------------------------------------------------------------------------------------------
+__device__ __forceinline__ float soft_cap(float y, float scale, float cap, float inv_cap) {
+  const float v = y * scale;
+  return cap > 0.f ? cap * tanhf(v * inv_cap) : v;
+}
+
+__global__ __launch_bounds__(256) void scale_soft_cap_kernel(float* __restrict__ y, long long n, float scale, float cap) {
+  const float inv_cap = cap > 0.f ? 1.f / cap : 0.f;
+  const long long i = ((long long)blockIdx.x * 256 + threadIdx.x) * 4;
+  if (i + 3 < n) {
+    float4 v = ld4(y + i);
+    v.x = soft_cap(v.x, scale, cap, inv_cap);
+    v.y = soft_cap(v.y, scale, cap, inv_cap);
+    v.z = soft_cap(v.z, scale, cap, inv_cap);
+    v.w = soft_cap(v.w, scale, cap, inv_cap);
+    st4(y + i, v);
+  } else {
+    for (long long e = i; e < n; ++e) y[e] = soft_cap(y[e], scale, cap, inv_cap);
+  }
+}
+
+extern "C" int sa_scale_soft_cap(float* y, long long n, float scale, float cap, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (!y || !(cap >= 0.f) || ((uintptr_t)y & 15)) return SA_ERR_ARG;
+  const long long blocks = (n + 1023) / 1024;
+  if (blocks > 0x7fffffffLL) return SA_ERR_ARG;
+  hipLaunchKernelGGL(scale_soft_cap_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, y, n, scale, cap);
   SA_LAUNCH_CHECK();
   return 0;
 }

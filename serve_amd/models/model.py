@@ -9,6 +9,7 @@ from typing import Dict, List, Optional, Tuple
 
 import torch
 
+from ..cache.retention import Retention
 from ..config.spec import ModelSpec, PartSpec
 from ..parts.base import LayerCache, Part, Runtime, StateRequest, TokenCacheRequest
 from ..registry import get_part
@@ -47,7 +48,11 @@ class Model:
             if not (set(roles) - optional) <= set(ls.parts) <= set(roles):
                 raise ValueError(f"layer {i}: arrangement {ls.arrangement!r} is built from the parts "
                                  f"{sorted(roles)}, the spec gives {sorted(ls.parts)}")
-            self.layers.append(arrangement(**{name: _make(roles[name], ps) for name, ps in ls.parts.items()}))
+            layer = arrangement(**{name: _make(roles[name], ps) for name, ps in ls.parts.items()})
+            biased = [n for n, p in layer.parts().items() if getattr(p, "has_output_bias", False)]
+            if biased and not getattr(arrangement, "adds_output_bias", False):
+                raise ValueError(f"layer {i}: arrangement {ls.arrangement!r} does not add the output bias of {biased}")
+            self.layers.append(layer)
         for e in spec.run_order:
             if not 0 <= e.layer < len(self.layers):
                 raise ValueError(f"run order names layer {e.layer}, the model has {len(self.layers)}")
@@ -144,15 +149,15 @@ class Model:
             elements, flops = elements + c.weight_elements, flops + c.flops
         return elements, flops
 
-    def cache_elements_per_token(self) -> List[Tuple[int, Optional[int]]]:
+    def cache_elements_per_token(self) -> List[Tuple[int, Retention]]:
         """Per cache layer that is read in a step (once per run-order entry that works on it):
-        (elements kept per token, window or None)."""
+        (elements kept per token, retention rule)."""
         reqs = self.cache_requests()
         out = []
         for e in self.spec.run_order:
             r = reqs[e.cache]
             if r is not None:
-                out.append((sum(t.elements_per_token() for t in r.tensors), r.window))
+                out.append((sum(t.elements_per_token() for t in r.tensors), r.retention))
         return out
 
     def graph_safe(self) -> bool:

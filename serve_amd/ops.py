@@ -113,16 +113,22 @@ def embed(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor,
 
 
 def add_rmsnorm(x: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
-                out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """x += delta (fp32 residual stream, in place), out = rmsnorm(x) * weight.
+                out: torch.Tensor, rows: Optional[torch.Tensor] = None,
+                after: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x += delta (fp32 residual stream, in place), out = rmsnorm(x) * weight; then x += after (fp32 [d], or None): a
+    constant row that joins the stream and that this norm does not see (not together with `rows`).
 
     `delta` is [T, d] in the activation dtype or fp32, or fp32 [parts, T, d]: partial sums of a
     product whose inner dimension was cut across workgroups; the parts are added in order.
     With `rows`, only the listed rows are produced (out[r] from source row rows[r]) and x is
     left as it was."""
-    _dev(x, delta, weight, out, rows)
+    _dev(x, delta, weight, out, rows, after)
     _check(x.dtype == torch.float32 and x.dim() == 2, "residual stream must be fp32 [T, d]")
     T, d = x.shape
+    if after is not None:
+        _f32vec(after, d, "the row that is added behind the norm")
+        _check(_aligned16(after), "the row that is added behind the norm must be 16-byte aligned")
+        _check(rows is None, "with rows the stream is left as it is: nothing can be added to it")
     _check(weight.shape == (d,), f"norm weight must be [{d}]")
     R = T if rows is None else rows.numel()
     if rows is not None:
@@ -139,7 +145,7 @@ def add_rmsnorm(x: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Te
         delta_code = _code(delta)
     lib = load_library("elementwise")
     _ret(lib.sa_add_rmsnorm(_ptr(x), _ptr(delta), c_int(delta_code), c_int(parts), _ptr(weight),
-                            c_int(_code(weight)), _ptr(out), c_int(_code(out)), _ptr(rows), c_float(eps),
+                            c_int(_code(weight)), _ptr(out), c_int(_code(out)), _ptr(rows), _ptr(after), c_float(eps),
                             c_int(R), c_int(T), c_int(d), _stream()), "add_rmsnorm")
     return out
 
@@ -242,17 +248,25 @@ def _check_sinks(sinks: Optional[torch.Tensor], num_heads: int) -> None:
                and sinks.numel() == num_heads, f"sinks must be contiguous fp32 [{num_heads}] on the GPU")
 
 
+def _check_mask(window: Optional[int], chunk: Optional[int]) -> None:
+    """Which of the keys up to its own a token sees: all; with `window` the last `window` of them; with `chunk` those of
+    its own run of `chunk` positions (counted from the sequence's position 0)."""
+    _check(not (window and chunk), "a mask is a window or a chunk, not both")
+    _check((window or 0) >= 0 and (chunk or 0) >= 0, "a window or a chunk holds at least the token itself")
+
+
 def paged_attention_simple(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, k_pages: torch.Tensor,
                            v_pages: torch.Tensor, block_table: torch.Tensor, cu_q: torch.Tensor,
                            ctx_len: torch.Tensor, seg_of_token: torch.Tensor, num_tokens: int,
                            num_heads: int, scale: float, window: Optional[int],
-                           sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                           sinks: Optional[torch.Tensor] = None, chunk: Optional[int] = None) -> torch.Tensor:
     """Attention of every token of the step over its request's cached keys (fp32 arithmetic), a wave
     per (token, head): the general form, for sizes that the other kernels do not take.
 
     q is the start of the q block of the fused qkv rows (row stride `q_row_stride` elements)."""
     _dev(q, out, k_pages, v_pages, block_table, cu_q, ctx_len, seg_of_token)
     _check_sinks(sinks, num_heads)
+    _check_mask(window, chunk)
     P, Hk, page_size, D = k_pages.shape
     _check(v_pages.shape == (P, Hk, D, page_size), "v_pages must be [P, Hk, D, page_size]")
     _check(num_heads % Hk == 0, "query heads must be a multiple of KV heads")
@@ -271,7 +285,7 @@ def paged_attention_simple(q: torch.Tensor, q_row_stride: int, out: torch.Tensor
         _ptr(q), c_int(q_row_stride), _ptr(out), c_int(_code(q)), _ptr(k_pages), _ptr(v_pages),
         c_int(_code(k_pages)), _ptr(block_table), c_int(block_table.shape[1]), _ptr(cu_q), _ptr(ctx_len),
         _ptr(seg_of_token), c_int(T), c_int(num_heads), c_int(Hk), c_int(D), c_int(page_size),
-        c_float(scale), c_int(window or 0), _ptr(sinks), _stream()), "paged_attention_simple")
+        c_float(scale), c_int(window or 0), c_int(chunk or 0), _ptr(sinks), _stream()), "paged_attention_simple")
     return out
 
 
@@ -286,7 +300,7 @@ def paged_attention_tiled_f32(q: torch.Tensor, q_row_stride: int, out: torch.Ten
                               v_pages: torch.Tensor, block_table: torch.Tensor, cu_q: torch.Tensor,
                               ctx_len: torch.Tensor, num_tokens: int, max_q_len: int, num_heads: int,
                               scale: float, window: Optional[int], num_splits: int = 1,
-                              sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                              sinks: Optional[torch.Tensor] = None, chunk: Optional[int] = None) -> torch.Tensor:
     """float32 attention: 64 rows (tokens x the query heads of a KV head) a workgroup share the keys
     and values of their KV head through LDS (fp32 arithmetic on the vector ALU).  `num_splits` > 1
     cuts the key range of every tile into that many parts across workgroups, merged by a second kernel
@@ -295,6 +309,7 @@ def paged_attention_tiled_f32(q: torch.Tensor, q_row_stride: int, out: torch.Ten
     to the end of the last of them, and only their rows of `out` are written."""
     _dev(q, out, k_pages, v_pages, block_table, cu_q, ctx_len)
     _check_sinks(sinks, num_heads)
+    _check_mask(window, chunk)
     P, Hk, page_size, D = k_pages.shape
     _check(tiled_attention_available(q, k_pages, q_row_stride),
            f"paged_attention_tiled_f32 takes float32, head sizes 16..128 in steps of 16 and page sizes that are "
@@ -319,7 +334,7 @@ def paged_attention_tiled_f32(q: torch.Tensor, q_row_stride: int, out: torch.Ten
     _ret(lib.sa_paged_attention_tiled_f32(
         _ptr(q), c_int(q_row_stride), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
         c_int(block_table.shape[1]), _ptr(cu_q), _ptr(ctx_len), c_int(B), c_int(T), c_int(max_q_len),
-        c_int(num_heads), c_int(Hk), c_int(D), c_int(page_size), c_float(scale), c_int(window or 0),
+        c_int(num_heads), c_int(Hk), c_int(D), c_int(page_size), c_float(scale), c_int(window or 0), c_int(chunk or 0),
         c_int(num_splits), _ptr(part_o), _ptr(part_ml), _ptr(sinks), _stream()), "paged_attention_tiled_f32")
     return out
 
@@ -328,7 +343,7 @@ def paged_attention_decode_f32(q: torch.Tensor, q_row_stride: int, out: torch.Te
                                v_pages: torch.Tensor, block_table: torch.Tensor, cu_q: torch.Tensor,
                                ctx_len: torch.Tensor, num_heads: int, scale: float, window: Optional[int],
                                num_splits: int = 1, first_token: int = 0,
-                               sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                               sinks: Optional[torch.Tensor] = None, chunk: Optional[int] = None) -> torch.Tensor:
     """float32 attention of B segments of one token each, a run of the step's tokens that begins at
     token `first_token` (the tables may be a slice of a longer step's; cu_q[i] must be first_token + i,
     which the caller knows on the host and the kernels do not check): a wave takes up to four query
@@ -336,6 +351,7 @@ def paged_attention_decode_f32(q: torch.Tensor, q_row_stride: int, out: torch.Te
     every key range into that many parts across workgroups, merged by a second kernel."""
     _dev(q, out, k_pages, v_pages, block_table, cu_q, ctx_len)
     _check_sinks(sinks, num_heads)
+    _check_mask(window, chunk)
     P, Hk, page_size, D = k_pages.shape
     _check(tiled_attention_available(q, k_pages, q_row_stride),
            f"paged_attention_decode_f32 takes float32, head sizes 16..128 in steps of 16 and page sizes that are "
@@ -363,7 +379,7 @@ def paged_attention_decode_f32(q: torch.Tensor, q_row_stride: int, out: torch.Te
     _ret(lib.sa_paged_attention_decode_f32(
         _ptr(q), c_int(q_row_stride), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
         c_int(block_table.shape[1]), _ptr(cu_q), _ptr(ctx_len), c_int(B), c_int(first_token), c_int(num_heads),
-        c_int(Hk), c_int(D), c_int(page_size), c_float(scale), c_int(window or 0), c_int(num_splits), _ptr(part_o),
+        c_int(Hk), c_int(D), c_int(page_size), c_float(scale), c_int(window or 0), c_int(chunk or 0), c_int(num_splits), _ptr(part_o),
         _ptr(part_ml), _ptr(sinks), _stream()), "paged_attention_decode_f32")
     return out
 
@@ -457,6 +473,34 @@ def activation(a: torch.Tensor, kind: str) -> torch.Tensor:
     _ret(lib.sa_activation(_ptr(a), c_int(_code(a)), ctypes.c_longlong(a.numel()), c_int(ACTIVATIONS[kind]),
                            _stream()), "activation")
     return a
+
+
+POLY_NORM_TERMS = 3
+
+
+def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float, out: torch.Tensor) -> torch.Tensor:
+    """out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 per row, powers element by element, N(y) = y / sqrt(mean(y^2) + eps);
+    z [T, n] in out's dtype or fp32, or fp32 [parts, T, n] partial sums that are added in order; coef fp32 [4]."""
+    _dev(z, coef, out)
+    _check(out.dim() == 2, "out must be [T, n]")
+    T, n = out.shape
+    parts = _parts_of(z, T, n, "z")
+    _check(z.dtype in (out.dtype, torch.float32), "z must have out's dtype or be fp32")
+    _f32vec(coef, POLY_NORM_TERMS + 1, "the coefficients")
+    lib = load_library("sublayer")
+    _ret(lib.sa_poly_norm(_ptr(z), c_int(_code(z)), c_int(parts), _ptr(coef), c_float(eps), _ptr(out), c_int(_code(out)),
+                          c_int(T), c_int(n), _stream()), "poly_norm")
+    return out
+
+
+def scale_soft_cap(y: torch.Tensor, scale: float, cap: float) -> torch.Tensor:
+    """y = cap tanh(scale y / cap) in place (cap 0: y = scale y); fp32, contiguous."""
+    _dev(y)
+    _check(y.dtype == torch.float32 and cap >= 0.0, "soft cap: fp32 values, a cap that is not negative")
+    lib = load_library("sublayer")
+    _ret(lib.sa_scale_soft_cap(_ptr(y), ctypes.c_longlong(y.numel()), c_float(scale), c_float(cap), _stream()),
+         "scale_soft_cap")
+    return y
 
 
 def sigmoid_mul(a: torch.Tensor, g: torch.Tensor) -> torch.Tensor:
@@ -581,18 +625,31 @@ def qk_norm_kv_write(qkv: torch.Tensor, q_out: torch.Tensor, positions: torch.Te
                      k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], q_weight: torch.Tensor,
                      k_weight: torch.Tensor, eps: float, num_heads: int, num_kv_heads: int, dim: int, vdim: int,
                      temp_coef: float = 0.0, temp_every: int = 0, v_first: Optional[torch.Tensor] = None,
-                     v_blend: float = 0.0) -> torch.Tensor:
-    """From rows qkv [T, Hq D | Hk D | Hk Dv]: every query and key head over its root mean square (eps inside
-    the root) times `q_weight` / `k_weight` (fp32 [D]); queries at position p times
+                     v_blend: float = 0.0, bias: Optional[torch.Tensor] = None,
+                     inv_freq: Optional[torch.Tensor] = None, rot_dim: int = 0,
+                     values_are_keys: bool = False) -> torch.Tensor:
+    """From rows qkv [T, Hq D | Hk D | Hk Dv] plus `bias` (fp32 over these columns, or None): every query and key head
+    over its root mean square (eps inside the root) times `q_weight` / `k_weight` (fp32 [D]), then its first `rot_dim`
+    dims rotated by position * inv_freq[i] (dim i paired with i + rot_dim / 2); queries at position p times
     1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) (temp_every 0: not); values blended as
     (1 - v_blend) v + v_blend v_first (v_first [T, >= Hk Dv] rows, may be a view with a row stride; None: not).
+    `values_are_keys`: the rows are [T, Hq D | Hk D], and a token's values are its keys as projected (with their
+    bias, before norm and rotation; Dv = D).
     Queries go to q_out [T, Hq Dp], keys and values to the token's slot of k_pages [P, Hk, page, Dp] and
     v_pages [P, Hk, Dp, page], each padded with zeros up to the cache's head size Dp.  `slots` None: queries only."""
-    _dev(q_out, positions, slots, k_pages, v_pages, q_weight, k_weight)
+    _dev(q_out, positions, slots, k_pages, v_pages, q_weight, k_weight, bias, inv_freq)
     Hq, Hk, D, Dv = num_heads, num_kv_heads, dim, vdim
     T = qkv.shape[0]
-    _check(qkv.is_cuda and qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= Hq * D + Hk * (D + Dv),
-           f"qkv must be rows of at least {Hq * D + Hk * (D + Dv)} on the GPU")
+    _check(not values_are_keys or D == Dv, "values that are the keys have the keys' size")
+    cols = Hq * D + Hk * D + (0 if values_are_keys else Hk * Dv)
+    _check(qkv.is_cuda and qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= cols,
+           f"qkv must be rows of at least {cols} on the GPU")
+    if bias is not None:
+        _f32vec(bias, cols, "bias")
+    _check(rot_dim >= 0 and rot_dim % 2 == 0 and rot_dim <= D, "rot_dim must be even and within dim")
+    if rot_dim:
+        _check(inv_freq is not None, "a rotation needs its frequencies")
+        _f32vec(inv_freq, rot_dim // 2, "inv_freq")
     _check(q_out.dim() == 2 and q_out.shape[0] == T and q_out.shape[1] % Hq == 0 and q_out.dtype == qkv.dtype,
            "q_out must be [T, Hq Dp] in the dtype of qkv")
     Dp = q_out.shape[1] // Hq
@@ -619,8 +676,9 @@ def qk_norm_kv_write(qkv: torch.Tensor, q_out: torch.Tensor, positions: torch.Te
                                  _ptr(slots), _ptr(k_pages if slots is not None else None),
                                  _ptr(v_pages if slots is not None else None), _ptr(q_weight), _ptr(k_weight),
                                  c_float(eps), c_float(temp_coef), c_int(temp_every), _ptr(v_first), c_int(vf_stride),
-                                 c_float(v_blend), c_int(T), c_int(Hq), c_int(Hk), c_int(D), c_int(Dv), c_int(Dp),
-                                 c_int(page_size), _stream()), "qk_norm_kv_write")
+                                 c_float(v_blend), _ptr(bias), _ptr(inv_freq if rot_dim else None), c_int(rot_dim),
+                                 c_int(1 if values_are_keys else 0), c_int(T), c_int(Hq), c_int(Hk), c_int(D), c_int(Dv),
+                                 c_int(Dp), c_int(page_size), _stream()), "qk_norm_kv_write")
     return q_out
 
 
@@ -871,11 +929,12 @@ def _rows(t: torch.Tensor, T: int, width: int, name: str) -> None:
 
 def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
                state_offset: int, ctx, out: torch.Tensor, heads: int, qk_heads: int, dk: int, dv: int,
-               q_scale: float = 1.0, piece_ok: bool = True) -> torch.Tensor:
+               q_scale: float = 1.0, piece_ok: bool = True, silu: bool = False) -> torch.Tensor:
     """Per segment of the step and head h, from the request's state S (fp32, zeros for a new request), token by token:
     S = diag(a) S + k v^T, out = S^T (q_scale q).  q, k: rows [T, >= qk_heads dk] (views with a row stride are fine;
     head h reads q/k head h // (heads / qk_heads)); v rows [T, >= heads dv]; all three of one dtype.  decay: ln a, fp32
-    [T, heads, dk] (one per key channel) or [T, heads] (one per head).  A step whose longest segment has
+    [T, heads, dk] (one per key channel), [T, heads] (one per head) or [heads] (one per head, the same for every token).
+    `silu`: q, k and v pass z sigmoid(z) as they are read.  A step whose longest segment has
     `SCAN_BLOCK_MIN_TOKENS` tokens or more takes sixteen tokens a pass on the matrix cores (keys up to 128 wide),
     any other goes token by token; long segments of a step that would leave most of the chip idle are cut into pieces
     that run side by side (`piece_ok` False: never).  state fp32 [slots, row]: the matrices live at
@@ -889,8 +948,9 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     _rows(v, T, heads * dv, "v")
     _check(q.dtype == k.dtype == v.dtype and q.device == k.device == v.device == out.device, "q, k and v must share dtype and device")
     per_channel = decay.dim() == 3
-    _check(decay.dtype == torch.float32 and tuple(decay.shape) in ((T, heads, dk), (T, heads)),
-           "decay must be fp32 [T, H, dk] or [T, H]")
+    _check(decay.dtype == torch.float32 and tuple(decay.shape) in ((T, heads, dk), (T, heads), (heads,)),
+           "decay must be fp32 [T, H, dk], [T, H] or [H]")
+    decay_stride = heads * dk if per_channel else (heads if decay.dim() == 2 else 0)
     _check(out.dtype == torch.float32 and out.shape == (T, heads * dv), "out must be fp32 [T, H dv]")
     need = decay_scan_state_floats(heads, dk, dv)
     _check(state.is_cuda and state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
@@ -918,7 +978,7 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
         else:
             piece = 0
     _ret(lib.sa_decay_scan(_ptr(q), _ptr(k), _ptr(v), c_int(_code(q)), LL(q.stride(0)), LL(k.stride(0)), LL(v.stride(0)),
-                           _ptr(decay), c_int(1 if per_channel else 0), c_float(q_scale),
+                           _ptr(decay), c_int(1 if per_channel else 0), LL(decay_stride), c_int(1 if silu else 0), c_float(q_scale),
                            c_void_p(state.data_ptr() + 4 * state_offset), LL(state.stride(0)), _ptr(ctx.cu_q),
                            _ptr(ctx.state_slots), _ptr(out), c_int(B), c_int(heads), c_int(qk_heads), c_int(dk), c_int(dv),
                            c_int(max_q), c_int(piece), _ptr(scratch), LL(scratch.stride(0) if scratch is not None else 0),
@@ -996,16 +1056,20 @@ def conv_state_update(zx: torch.Tensor, col: int, channels: int, state: torch.Te
                                   c_int(taps), _stream()), "conv_state_update")
 
 
+READOUT_GATES = {"silu": 0, "sigmoid": 1}
+
+
 def gated_group_norm(o: torch.Tensor, gate_rows: torch.Tensor, gate_col: int, weight: torch.Tensor, group: int,
                      gate_first: bool, eps: float, out: torch.Tensor, skip_x: Optional[torch.Tensor] = None,
-                     skip_d: Optional[torch.Tensor] = None, head_dim: int = 1) -> torch.Tensor:
+                     skip_d: Optional[torch.Tensor] = None, head_dim: int = 1, gate: str = "silu") -> torch.Tensor:
     """What follows a recurrence's read-out o fp32 [T, n]: u = o + skip_d[i // head_dim] skip_x[t, i] (skip_x fp32 rows
-    [T, >= n], or None); with g = silu(gate_rows[t, gate_col + i]): `gate_first`: out = N(u g) w, else out = N(u) w g,
+    [T, >= n], or None); with g = silu(gate_rows[t, gate_col + i]) (`gate` "sigmoid": the sigmoid of it): `gate_first`: out = N(u g) w, else out = N(u) w g,
     where N divides every run of `group` values by its root mean square (eps inside the root) and w = weight[i % len]."""
     _dev(o, weight, out, skip_d)
     _check(o.dtype == torch.float32 and o.dim() == 2, "o must be fp32 [T, n]")
     T, n = o.shape
     _check(group > 0 and n % group == 0, f"groups of {group} do not divide {n}")
+    _check(gate in READOUT_GATES, f"unknown gate {gate!r}; known: {sorted(READOUT_GATES)}")
     _check(out.shape == (T, n) and out.dtype == gate_rows.dtype, "out must be [T, n] in the gate's dtype")
     _rows(gate_rows, T, gate_col + n, "gate rows")
     _check(weight.dtype == torch.float32 and weight.dim() == 1 and weight.numel() > 0, "the norm's weight must be an fp32 vector")
@@ -1019,8 +1083,46 @@ def gated_group_norm(o: torch.Tensor, gate_rows: torch.Tensor, gate_col: int, we
     LL = ctypes.c_longlong
     _ret(lib.sa_gated_group_norm(_ptr(o), _ptr(skip_x), LL(skip_stride), _ptr(skip_d), c_int(head_dim), _ptr(gate_rows),
                                  c_int(_code(gate_rows)), LL(gate_rows.stride(0)), c_int(gate_col), _ptr(weight),
-                                 c_int(weight.numel()), c_int(group), c_int(1 if gate_first else 0), c_float(eps), _ptr(out),
+                                 c_int(weight.numel()), c_int(group), c_int(1 if gate_first else 0), c_int(READOUT_GATES[gate]),
+                                 c_float(eps), _ptr(out),
                                  c_int(T), c_int(n), _stream()), "gated_group_norm")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------
+# element-wise gated averages S_t = (1 - z_t) S_(t-1) + z_t c_t
+# ---------------------------------------------------------------------------------------------
+GATED_AVERAGE_TILE = 32          # tokens a workgroup takes (csrc/gated_average.hip: GA_TILE)
+GATED_AVERAGE_SHORT = 16         # steps whose longest segment has at most this many tokens go segment by segment
+
+
+def gated_average(rows: torch.Tensor, bias: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor) -> torch.Tensor:
+    """Per segment of the step and channel, from the request's state S (fp32 [slots, >= W], zeros for a new request):
+    with rows fp32 [T, 3 W] = [z | u | g] (or [parts, T, 3 W] partial sums that are added in order) and bias fp32 [2 W]
+    (z's, then u's): z = sigmoid(z + b_z); c = u + 1/2 where u + b_u >= 0, else sigmoid(u) (u with its bias);
+    S = (1 - z) S + z c; out[t] = S silu(g).  All arithmetic is fp32; out [T, W] in any kernel dtype."""
+    T, B = ctx.num_tokens, ctx.num_segments
+    _dev(rows, bias, out, ctx.cu_q, ctx.seg_of_token, ctx.state_slots)
+    _check(out.dim() == 2 and out.shape[0] == T, "out must be [T, W]")
+    W = out.shape[1]
+    _check(rows.dtype == torch.float32, "what enters the recurrence must be fp32")
+    parts = _parts_of(rows, T, 3 * W, "rows")
+    _f32vec(bias, 2 * W, "bias")
+    _check(state.is_cuda and state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+           and state.shape[1] >= W, f"state rows must be fp32 with {W} floats")
+    _i32(ctx.cu_q, B + 1, "cu_q")
+    _i32(ctx.seg_of_token, T, "seg_of_token")
+    _i32(ctx.state_slots, B, "state_slots")
+    lib = load_library("gated_average")
+    max_q = int(getattr(ctx, "max_q_len", 0) or T)
+    by_segment = max_q <= GATED_AVERAGE_SHORT
+    scratch = None
+    if not by_segment and T > GATED_AVERAGE_TILE:
+        scratch = torch.empty((-(-T // GATED_AVERAGE_TILE), 3 * W), dtype=torch.float32, device=out.device)
+    _ret(lib.sa_gated_average(_ptr(rows), c_int(parts), _ptr(bias), _ptr(state), ctypes.c_longlong(state.stride(0)),
+                              _ptr(ctx.cu_q), _ptr(ctx.seg_of_token), _ptr(ctx.state_slots), _ptr(out), c_int(_code(out)),
+                              _ptr(scratch), c_int(T), c_int(B), c_int(W), c_int(1 if by_segment else 0), _stream()),
+         "gated_average")
     return out
 
 
@@ -1459,7 +1561,7 @@ def paged_attention_mfma(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, 
                          ctx_len: torch.Tensor, num_tokens: int, max_q_len: int, num_heads: int, scale: float,
                          window: Optional[int], num_splits: int = 1, seg_begin: int = 0,
                          seg_count: Optional[int] = None, in_workgroup: bool = False,
-                         sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                         sinks: Optional[torch.Tensor] = None, chunk: Optional[int] = None) -> torch.Tensor:
     """bf16 attention on the matrix cores (head sizes 16..128 in steps of 16, page sizes that are
     multiples of 4).  `in_workgroup` (segments of at most 16 rows per KV head, num_splits 1): the
     key range is cut four ways over the waves of a workgroup, which merges the parts itself.  `seg_begin`, `seg_count`: run only these segments of the step (their
@@ -1467,6 +1569,7 @@ def paged_attention_mfma(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, 
     tokens up to the end of the last of them."""
     _dev(q, out, k_pages, v_pages, block_table, cu_q, ctx_len)
     _check_sinks(sinks, num_heads)
+    _check_mask(window, chunk)
     P, Hk, page_size, D = k_pages.shape
     _check(mfma_attention_available(q, k_pages, q_row_stride, scale),
            f"paged_attention_mfma takes bf16, head sizes {MFMA_ATTENTION_HEAD_DIMS}, page sizes that are "
@@ -1504,7 +1607,7 @@ def paged_attention_mfma(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, 
     _ret(lib.sa_paged_attention_mfma(
         _ptr(q), c_int(q_row_stride), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
         c_int(block_table.shape[1]), _ptr(cu_q), _ptr(ctx_len), c_int(B), c_int(T), c_int(max_q_len),
-        c_int(num_heads), c_int(Hk), c_int(D), c_int(page_size), c_float(scale), c_int(window or 0),
+        c_int(num_heads), c_int(Hk), c_int(D), c_int(page_size), c_float(scale), c_int(window or 0), c_int(chunk or 0),
         c_int(num_splits), _ptr(part_o), _ptr(part_ml), c_int(1 if in_workgroup else 0), _ptr(sinks), _stream()),
         "paged_attention_mfma")
     return out
@@ -1558,36 +1661,45 @@ def _attention_launches(ctx):
     return plan
 
 
+def _keys_in_reach(max_ctx: int, max_q: int, window: Optional[int], chunk: Optional[int]) -> int:
+    """The most keys that a launch's segments read: a mask that reaches back only so far bounds them."""
+    reach = window or chunk
+    return min(max_ctx, reach + max_q - 1) if reach else max_ctx
+
+
 def paged_attention(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, k_pages: torch.Tensor,
                     v_pages: torch.Tensor, block_table: torch.Tensor, ctx, num_heads: int, scale: float,
-                    window: Optional[int], sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    window: Optional[int], sinks: Optional[torch.Tensor] = None,
+                    chunk: Optional[int] = None) -> torch.Tensor:
     """Attention over the paged cache for all tokens of the step described by `ctx` (an `AttentionStep`,
     or anything with its attributes: the engine passes its `StepContext`): the matrix-core kernel for
     bf16 where it takes the sizes, else the general fp32-arithmetic kernel.  The plan of launches is
     kept on `ctx`, so that the layers of a step share it.  `sinks` (fp32 [Hq]): one more term exp(sinks[h])
-    in the denominator of head h's softmax, in every kernel."""
+    in the denominator of head h's softmax, in every kernel.  `window` / `chunk` (at most one): see `_check_mask`."""
     if mfma_attention_available(q, k_pages, q_row_stride, scale):
         Hk = k_pages.shape[1]
         # (first segment, segments, tokens up to their end, longest portion, longest context)
         for s0, n, t_end, max_q, max_ctx in _attention_launches(ctx):
             # (the parts of a split key range are indexed by token, from the step's first)
+            max_ctx = _keys_in_reach(max_ctx, max_q, window, chunk)
             inside = max_q == 1 and attention_in_workgroup(max_q, n, max_ctx, num_heads // Hk)
             splits = 1
             if not inside and (max_q == 1 or s0 == 0):
                 splits = attention_splits(max_q, n, Hk, max_ctx, num_heads // Hk)
             paged_attention_mfma(q, q_row_stride, out, k_pages, v_pages, block_table, ctx.cu_q, ctx.ctx_len,
                                  t_end, max_q, num_heads, scale, window, splits, s0, n, in_workgroup=inside,
-                                 sinks=sinks)
+                                 sinks=sinks, chunk=chunk)
         return out
     Hk = k_pages.shape[1]
     if tiled_attention_available(q, k_pages, q_row_stride):
         G = num_heads // Hk
         launches = _attention_launches(ctx)
         if len(launches) > 1 or ctx.max_q_len == 1 or ctx.max_q_len * G > TILED_MIN_ROWS \
-                or ctx.max_ctx_len >= TILED_MIN_CONTEXT:
+                or _keys_in_reach(ctx.max_ctx_len, ctx.max_q_len, window, chunk) >= TILED_MIN_CONTEXT:
             # decoding requests and prompt portions as two launches, as on the matrix-core path
             for s0, n, t_end, max_q, max_ctx in launches:
                 whole = s0 == 0 and n == ctx.num_segments
+                max_ctx = _keys_in_reach(max_ctx, max_q, window, chunk)
                 bt = block_table if whole else block_table[s0: s0 + n]
                 cu = ctx.cu_q if whole else ctx.cu_q[s0: s0 + n + 1]
                 cl = ctx.ctx_len if whole else ctx.ctx_len[s0: s0 + n]
@@ -1597,14 +1709,14 @@ def paged_attention(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, k_pag
                     waves = n * Hk * -(-G // 4)
                     splits = max(1, min(64, FP32_DECODE_WAVES // max(waves, 1), max_ctx // 128))
                     paged_attention_decode_f32(q, q_row_stride, out, k_pages, v_pages, bt, cu, cl, num_heads, scale,
-                                               window, splits, sinks=sinks)
+                                               window, splits, sinks=sinks, chunk=chunk)
                     continue
                 splits = 1
                 if max_q * G <= TILED_MIN_ROWS and max_ctx >= TILED_MIN_CONTEXT and s0 == 0:
                     # few rows over many keys: about two workgroups per compute unit, parts of at least 256 keys
                     splits = max(1, min(64, 2 * compute_units() // max(n * Hk, 1), max_ctx // 256))
                 paged_attention_tiled_f32(q, q_row_stride, out, k_pages, v_pages, bt, cu, cl, t_end, max_q,
-                                          num_heads, scale, window, splits, sinks=sinks)
+                                          num_heads, scale, window, splits, sinks=sinks, chunk=chunk)
             return out
     return paged_attention_simple(q, q_row_stride, out, k_pages, v_pages, block_table, ctx.cu_q,
-                                  ctx.ctx_len, ctx.seg_of_token, ctx.num_tokens, num_heads, scale, window, sinks)
+                                  ctx.ctx_len, ctx.seg_of_token, ctx.num_tokens, num_heads, scale, window, sinks, chunk)

@@ -9,13 +9,16 @@ Roles and what each must offer:
 * norm          `forward(x, delta, rows=None) -> y`: adds `delta` (or nothing) into the fp32
                 residual stream `x` in place and returns the normalised activations in the
                 activation dtype; with `rows` it returns only those rows and leaves x alone.
-                `delta` is [T, d], or fp32 [parts, T, d] partial sums to be added in order.
+                `delta` is [T, d], or fp32 [parts, T, d] partial sums to be added in order.  With
+                `after=` (fp32 [d]; not with `rows`) that row joins the stream behind the norm.
 * position      owned by a mixer, which asks it either for a rotation it can hand to its fused
                 kernels (`rotary()`) or to encode q and k itself (`apply(q, k, positions)`); it
                 never touches the cache: the mixer stores what it keeps.
 * mixer         `forward(h, ctx, cache, writes_cache) -> delta [T, d]`; may ask for per-token
                 cache (`cache_request`: a list of tensors per token and a retention rule) and
-                for per-request state of fixed size (`state_request`).
+                for per-request state of fixed size (`state_request`).  A mixer whose output has a
+                bias leaves it in `output_bias` (fp32 [d]) when it loads and says so before with
+                `has_output_bias`: the arrangement adds it to the stream (those that do: `adds_output_bias`).
 * feed_forward  `forward(h, ctx) -> delta [T, d]`.
 * embedding     `forward(ctx) -> x` fp32 [T, d] from the step's token ids (and whatever else of
                 the step it needs: positions for a learned position table).  An embedding that looks
@@ -34,6 +37,8 @@ from dataclasses import dataclass
 from typing import Dict, List, Optional, Tuple
 
 import torch
+
+from ..cache.retention import Chunks, Retention
 
 
 @dataclass(frozen=True)
@@ -84,19 +89,38 @@ class CacheTensor:
 @dataclass(frozen=True)
 class TokenCacheRequest:
     """Per-token cache a mixer needs in its layer: the tensors it keeps for every token, for the
-    whole context (`window=None`) or for the last `window` tokens."""
+    whole context, for the last `window` tokens, or for the current run of `chunk` positions."""
 
     tensors: Tuple[CacheTensor, ...]
     window: Optional[int] = None
+    chunk: Optional[int] = None
+
+    def __post_init__(self):
+        if self.window is not None and self.chunk is not None:
+            raise ValueError("a cache keeps a window or a chunk, not both")
+
+    @property
+    def retention(self) -> Retention:
+        return self.window if self.chunk is None else Chunks(self.chunk)
 
 
-def kv_cache_request(num_kv_heads: int, head_dim: int, window: Optional[int] = None) -> TokenCacheRequest:
+def kv_cache_request(num_kv_heads: int, head_dim: int, window: Optional[int] = None,
+                     chunk: Optional[int] = None) -> TokenCacheRequest:
     """Keys and values of `num_kv_heads` heads of `head_dim` as the attention kernels read them:
     keys [P, Hk, page, D] (one head's keys of a page are contiguous rows), values
     [P, Hk, D, page] (transposed inside the page, so that the matrix-core product P.V reads runs
     of consecutive keys at a fixed dim)."""
     return TokenCacheRequest((CacheTensor("k", (num_kv_heads, head_dim), 1),
-                              CacheTensor("v", (num_kv_heads, head_dim), 2)), window)
+                              CacheTensor("v", (num_kv_heads, head_dim), 2)), window, chunk)
+
+
+def keys_seen(tokens: int, context_before: int, window: Optional[int] = None, chunk: Optional[int] = None) -> int:
+    """Keys that `tokens` tokens behind a context of `context_before` see in all (for accounts of flops)."""
+    if chunk:
+        return sum((context_before + j) % chunk + 1 for j in range(tokens))
+    if window:
+        return sum(min(context_before + j + 1, window) for j in range(tokens))
+    return tokens * context_before + tokens * (tokens + 1) // 2
 
 
 @dataclass(frozen=True)
@@ -164,6 +188,10 @@ class Part:
     # whether `forward` only enqueues GPU work on the current stream (no read-back to the host,
     # no host-side branching on device data): only then can a step be captured into a HIP graph
     graph_safe = False
+
+    # a constant row that belongs to this part's output and that its arrangement adds to the residual stream
+    has_output_bias = False
+    output_bias: Optional[torch.Tensor] = None
 
     def param_requests(self) -> List[ParamRequest]:
         return []

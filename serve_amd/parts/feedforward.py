@@ -15,25 +15,36 @@ from .standard import SwiGLU, _prepare_products
 
 
 class DenseFeedForward(Part):
-    """down(act(up x)), no biases; act = one of `ops.ACTIVATIONS` ('gelu_tanh', 'silu', 'relu_squared')."""
+    """down(act(up x)), no biases; act = one of `ops.ACTIVATIONS` ('gelu_tanh', 'silu', 'relu_squared'), or 'poly_norm'
+    with the four stored numbers of `act`: a N(z) + b N(z^2) + c N(z^3) + e, powers element by element, N(y) = y over the
+    root mean square of the token's values (`eps` inside the root)."""
 
     graph_safe = True
 
-    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "gelu_tanh"):
-        if activation not in ops.ACTIVATIONS:
-            raise ValueError(f"unknown activation {activation!r}; known: {sorted(ops.ACTIVATIONS)}")
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "gelu_tanh", eps: float = 0.0):
+        if activation not in ops.ACTIVATIONS and activation != "poly_norm":
+            raise ValueError(f"unknown activation {activation!r}; known: {sorted(ops.ACTIVATIONS) + ['poly_norm']}")
         self.hidden_size, self.intermediate_size, self.activation = int(hidden_size), int(intermediate_size), activation
+        self.eps = float(eps)
 
     def param_requests(self) -> List[ParamRequest]:
         d, i = self.hidden_size, self.intermediate_size
-        return [ParamRequest("up", (i, d), init="normal:0.07"), ParamRequest("down", (d, i), init="normal:0.07")]
+        out = [ParamRequest("up", (i, d), init="normal:0.07"), ParamRequest("down", (d, i), init="normal:0.07")]
+        if self.activation == "poly_norm":
+            out.append(ParamRequest("act", (ops.POLY_NORM_TERMS + 1,), init="normal:0.4"))
+        return out
 
     def load(self, tensors, rt: Runtime) -> None:
         self.rt = rt
         self.w_up, self.w_down = tensors["up"], tensors["down"]
+        self.coef = tensors["act"].float().contiguous() if self.activation == "poly_norm" else None
         _prepare_products(rt, self.w_up)
 
     def forward(self, h: torch.Tensor, ctx) -> torch.Tensor:
+        if self.coef is not None:
+            z = linear(h, self.w_up, partial_ok=True)      # (few rows: fp32 sums, which the activation adds)
+            a = ops.poly_norm(z, self.coef, self.eps, self.rt.empty((h.shape[0], self.intermediate_size)))
+            return linear(a, self.w_down, partial_ok=True)
         a = ops.activation(linear(h, self.w_up), self.activation)
         return linear(a, self.w_down, partial_ok=True)
 

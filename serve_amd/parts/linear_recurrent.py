@@ -6,6 +6,10 @@
 channel a = sigmoid(W_a2 (W_a1 h) + b)^(1/tau); the read-out of every head over its root mean square, times a weight
 shared by the heads, times silu(W_g h), then W_o.
 
+`DecayedLinearAttention` (the form known as lightning attention): q = silu(W_q h), k = silu(W_k h) (heads x dim),
+v = silu(W_v h) (heads x vdim); one constant decay per head, given; the read-outs of all heads together over their root
+mean square, times a weight, times sigmoid(W_g h), then W_o.
+
 `StateSpaceMixer` (the selective state-space mixer in its state-space-duality form): W_in h = [z | x | B | C | dt] with
 inner = heads * vdim, B and C of groups * state; x, B, C pass a causal convolution per channel (`conv` taps, bias) and
 silu; dt = softplus(dt + dt_bias); per head S [state, vdim] with a = exp(-exp(A_log) dt), k = B, v = dt x, q = C
@@ -19,7 +23,7 @@ from products with fp32 results.
 """
 from __future__ import annotations
 
-from typing import List, Optional
+from typing import List, Optional, Sequence
 
 import torch
 
@@ -93,6 +97,56 @@ class GatedLinearAttention(Part):
         return linear(y, self.wo, partial_ok=True)
 
 
+class DecayedLinearAttention(Part):
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, decay: Sequence[float], eps: float):
+        if not (0 < dim <= ops.SCAN_MAX_DIM and vdim > 0 and heads > 0):
+            raise ValueError(f"key sizes up to {ops.SCAN_MAX_DIM} are taken; got heads {heads}, dim {dim}, vdim {vdim}")
+        self.decay = tuple(float(a) for a in decay)
+        if len(self.decay) != heads or not all(0.0 < a <= 1.0 for a in self.decay):
+            raise ValueError(f"one decay in (0, 1] per head is needed, got {list(self.decay)} for {heads} heads")
+        self.hidden_size, self.heads, self.dim, self.vdim, self.eps = int(hidden_size), int(heads), int(dim), int(vdim), float(eps)
+
+    def param_requests(self) -> List[ParamRequest]:
+        d, H, D, Dv = self.hidden_size, self.heads, self.dim, self.vdim
+        return [ParamRequest("q", (H * D, d), init="normal:0.08"), ParamRequest("k", (H * D, d), init="normal:0.08"),
+                ParamRequest("v", (H * Dv, d), init="normal:0.08"), ParamRequest("g", (H * Dv, d), init="normal:0.08"),
+                ParamRequest("o", (d, H * Dv), init="normal:0.08"), ParamRequest("norm", (H * Dv,), init="ones_normal:0.15")]
+
+    def state_request(self) -> StateRequest:
+        return StateRequest((ops.decay_scan_state_floats(self.heads, self.dim, self.vdim),), torch.float32)
+
+    def step_cost(self, tokens: int, context_before: int = 0) -> StepCost:
+        """The projections, and per token and head the decay with the outer product and the read-out: 4 dim vdim flops."""
+        cost = super().step_cost(tokens, context_before)
+        cost.flops += 4.0 * tokens * self.heads * self.dim * self.vdim
+        return cost
+
+    def load(self, tensors, rt: Runtime) -> None:
+        self.rt = rt
+        big = [tensors[n] for n in ("q", "k", "v", "g")]
+        dt = _same_dtype(big)
+        self.w_in = torch.cat([t.to(dt) for t in big], dim=0).contiguous()        # one product: q | k | v | gate
+        self.log_decay = torch.tensor(self.decay, dtype=torch.float64).log().float().to(rt.device)
+        self.norm_w = tensors["norm"].float().contiguous()
+        self.wo = tensors["o"]
+        _prepare_products(rt, self.w_in)
+
+    def forward(self, h: torch.Tensor, ctx, cache: LayerCache, writes_cache: bool = True) -> torch.Tensor:
+        if cache.state is None:
+            raise ValueError("the linear attention needs its per-request state")
+        H, D, Dv = self.heads, self.dim, self.vdim
+        T, v0, g0 = h.shape[0], 2 * H * D, 2 * H * D + H * Dv
+        z = linear(h, self.w_in)
+        o = torch.empty((T, H * Dv), dtype=torch.float32, device=h.device)
+        ops.decay_scan(z[:, : H * D], z[:, H * D: v0], z[:, v0: g0], self.log_decay, cache.state, 0, ctx, o, H, H, D, Dv,
+                       silu=True)
+        y = self.rt.empty((T, H * Dv))
+        ops.gated_group_norm(o, z, g0, self.norm_w, H * Dv, False, self.eps, y, gate="sigmoid")
+        return linear(y, self.wo, partial_ok=True)
+
+
 class StateSpaceMixer(Part):
     graph_safe = True
 
@@ -162,4 +216,5 @@ class StateSpaceMixer(Part):
 
 
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+register_part("mixer", "decayed_linear_attention", DecayedLinearAttention)
 register_part("mixer", "state_space", StateSpaceMixer)

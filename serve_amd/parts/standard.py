@@ -49,11 +49,11 @@ class RMSNorm(Part):
         # (for kernels that apply this norm at the end of another kernel's work and take fp32 vectors)
         self.weight_f32 = self.weight if self.weight.dtype == torch.float32 else self.weight.float()
 
-    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor],
-                rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor], rows: Optional[torch.Tensor] = None,
+                after: Optional[torch.Tensor] = None) -> torch.Tensor:
         n = x.shape[0] if rows is None else rows.numel()
         out = self.rt.empty((n, self.size))
-        return ops.add_rmsnorm(x, delta, self.weight, self.eps, out, rows)
+        return ops.add_rmsnorm(x, delta, self.weight, self.eps, out, rows, after)
 
 
 # ---------------------------------------------------------------------------------------------
@@ -71,8 +71,14 @@ def rope_inverse_frequencies(head_dim_rot: int, theta: float, scaling: Optional[
     kind = scaling.get("rope_type", scaling.get("type", "llama3"))
     if kind == "yarn":
         return yarn_frequencies(head_dim_rot, theta, scaling)[0]
+    if kind == "linear":
+        # every frequency divided by the factor; float64, rounded once
+        if not float(scaling["factor"]) > 0:
+            raise ValueError("linear scaling needs a positive factor")
+        i = torch.arange(head_dim_rot // 2, dtype=torch.float64)
+        return (float(theta) ** (-2.0 * i / head_dim_rot) / float(scaling["factor"])).float()
     if kind != "llama3":
-        raise ValueError(f"rope scaling {kind!r} is not supported (known: 'llama3', 'yarn')")
+        raise ValueError(f"rope scaling {kind!r} is not supported (known: 'llama3', 'yarn', 'linear')")
     factor = float(scaling["factor"])
     low = float(scaling["low_freq_factor"])
     high = float(scaling["high_freq_factor"])
@@ -124,8 +130,8 @@ class RotaryPosition(PositionPart):
     (serve/hf_utils/convert_hf_checkpoint.py:115-118), which is `pairing="adjacent"`.
     `rot_dim < head_dim` leaves the remaining dims of every head as they are.  The part only
     says what the rotation is (`rotary()`); the attention's kernels carry it out, fused with
-    the projection or the cache write.  `scaling` with `rope_type` "llama3" or "yarn" (see
-    `rope_inverse_frequencies`, `yarn_frequencies`); the latter also gives the rotation a magnitude."""
+    the projection or the cache write.  `scaling` with `rope_type` "llama3", "yarn" or "linear" (see
+    `rope_inverse_frequencies`, `yarn_frequencies`); "yarn" also gives the rotation a magnitude."""
 
     graph_safe = True
 
@@ -347,8 +353,12 @@ class LinearHead(Part):
     graph_safe = True
 
     def __init__(self, vocab_size: int, hidden_size: int, tied: bool = False,
-                 shares: Optional[str] = "embedding.weight"):
+                 shares: Optional[str] = "embedding.weight", scale: float = 1.0, soft_cap: float = 0.0):
+        """`scale` multiplies the products; `soft_cap` > 0 then keeps them within it: cap tanh(logit / cap)."""
         self.vocab_size, self.hidden_size, self.tied = int(vocab_size), int(hidden_size), bool(tied)
+        self.scale, self.soft_cap = float(scale), float(soft_cap)
+        if self.soft_cap < 0:
+            raise ValueError("a soft cap is positive, or 0 for none")
         self.shares = shares
         if self.tied and not shares:
             raise ValueError("a tied head needs the name of the tensor it shares")
@@ -369,7 +379,10 @@ class LinearHead(Part):
         if out is not None and (out.shape != (h.shape[0], self.vocab_size) or out.dtype != torch.float32
                                 or not out.is_contiguous()):
             raise ValueError(f"the logits buffer must be contiguous fp32 [{h.shape[0]}, {self.vocab_size}]")
-        return linear(h, self.weight, out_dtype=torch.float32, out=out)
+        y = linear(h, self.weight, out_dtype=torch.float32, out=out)
+        if self.scale != 1.0 or self.soft_cap:
+            ops.scale_soft_cap(y, self.scale, self.soft_cap)
+        return y
 
 
 # ---------------------------------------------------------------------------------------------
@@ -381,6 +394,9 @@ class PreNormResidual:
     The additions are folded into the following norm: `pending` is the output of the previous
     part that has not been added to the residual stream yet; the layer returns its own.
 
+    A bias of the mixer's output is a constant row: the mixer's norm adds it to the stream behind itself, which is where
+    the mixer's output joins it too.
+
     A layer may have no feed-forward (then it has no `ffn_norm` either), and it may end with a
     `token_input`: a part that adds something made from the step's tokens and the finished stream
     (`forward(x, pending, ctx) -> pending`: it folds the layer's last output into x itself).  Such a part may
@@ -390,10 +406,13 @@ class PreNormResidual:
     PART_ROLES = {"mixer": "mixer", "ffn": "feed_forward", "mixer_norm": "norm", "ffn_norm": "norm",
                   "token_input": "token_input"}
     OPTIONAL_PARTS = ("ffn", "ffn_norm", "token_input")
+    adds_output_bias = True
 
     def __init__(self, mixer, mixer_norm, ffn=None, ffn_norm=None, token_input=None):
         if (ffn is None) != (ffn_norm is None):
             raise ValueError("a feed-forward and its norm come together")
+        if any(p is not None and p.has_output_bias for p in (ffn, token_input)):
+            raise ValueError("this arrangement adds the mixer's output bias, and no other part's")
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
         self.token_input = token_input
 
@@ -417,6 +436,10 @@ class PreNormResidual:
         ready = ctx.shared.pop(NORMED_STREAM, None) if getattr(ctx, "shared", None) else None
         if ready is not None and ready[1] is self.mixer_norm and pending is None:
             h = ready[0]                            # the layer before has made it, with this layer's norm
+            if self.mixer.output_bias is not None:
+                ops.stream_add(x, None, self.mixer.output_bias)
+        elif self.mixer.output_bias is not None:
+            h = self.mixer_norm.forward(x, pending, after=self.mixer.output_bias)
         else:
             h = self.mixer_norm.forward(x, pending)
         a = self.mixer.forward(h, ctx, cache, writes_cache)

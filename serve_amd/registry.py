@@ -87,3 +87,4 @@ def _ensure_builtin() -> None:
         from .models import timopel  # noqa: F401  (registers Timopel)
         from .models import kotipel  # noqa: F401  (registers Kotipel)
         from .models import robuvik  # noqa: F401  (registers Robuvik)
+        from .models import topapel  # noqa: F401  (registers Topapel)
