@@ -31,7 +31,7 @@ class DenseFeedForward(Part):
         d, i = self.hidden_size, self.intermediate_size
         out = [ParamRequest("up", (i, d), init="normal:0.07"), ParamRequest("down", (d, i), init="normal:0.07")]
         if self.activation == "poly_norm":
-            out.append(ParamRequest("act", (ops.POLY_NORM_TERMS + 1,), init="normal:0.4"))
+            out.append(ParamRequest("act", (ops.POLY_NORM_TERMS + 1,), init="ones_normal:0.4"))
         return out
 
     def load(self, tensors, rt: Runtime) -> None:

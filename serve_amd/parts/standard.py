@@ -411,7 +411,7 @@ class PreNormResidual:
     def __init__(self, mixer, mixer_norm, ffn=None, ffn_norm=None, token_input=None):
         if (ffn is None) != (ffn_norm is None):
             raise ValueError("a feed-forward and its norm come together")
-        if any(p is not None and p.has_output_bias for p in (ffn, token_input)):
+        if any(getattr(p, "has_output_bias", False) for p in (ffn, token_input)):
             raise ValueError("this arrangement adds the mixer's output bias, and no other part's")
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
         self.token_input = token_input
@@ -434,12 +434,13 @@ class PreNormResidual:
     def forward(self, x: torch.Tensor, pending: Optional[torch.Tensor], ctx, cache: LayerCache,
                 writes_cache: bool = True) -> Optional[torch.Tensor]:
         ready = ctx.shared.pop(NORMED_STREAM, None) if getattr(ctx, "shared", None) else None
+        bias = getattr(self.mixer, "output_bias", None)
         if ready is not None and ready[1] is self.mixer_norm and pending is None:
             h = ready[0]                            # the layer before has made it, with this layer's norm
-            if self.mixer.output_bias is not None:
-                ops.stream_add(x, None, self.mixer.output_bias)
-        elif self.mixer.output_bias is not None:
-            h = self.mixer_norm.forward(x, pending, after=self.mixer.output_bias)
+            if bias is not None:
+                ops.stream_add(x, None, bias)
+        elif bias is not None:
+            h = self.mixer_norm.forward(x, pending, after=bias)
         else:
             h = self.mixer_norm.forward(x, pending)
         a = self.mixer.forward(h, ctx, cache, writes_cache)
