@@ -156,9 +156,33 @@ SHAPES.update({
     "robuvik-2k": _robuvik_shape(2048, 32768, 6, (2, 4, 2), 32, 8, 64, 1024, 512, 8192, 32, 4, 1024, 2048, 65521),
     "robuvik-4k": _robuvik_shape(4096, 32768, 3, (1, 2, 2), 32, 8, 128, 1024, 1024, 14336, 64, 6, 1536, 3072, 65521),
 })
+
+
+def _topapel_shape(width: int, vocab: int, layers: int, heads: int, kv_heads: int, head: int, chunk: int, gru: int,
+                   lin_heads: int, lin_dim: int, ff: int):
+    """A Topapel shape at the sizes of a real model's layers: in turn an attention layer (`heads` on `kv_heads` heads of
+    `head`, all dims rotated, chunks of `chunk`), a gated average of `gru` channels and a linear attention of `lin_heads`
+    heads of `lin_dim` x `lin_dim` with decays from 0.9 to 0.999, each with a feed-forward of `ff`."""
+    from .config.topapel import (ChunkAttentionConfig, LightningConfig, LinearRotConfig, MinGruConfig, TopapelConfig,
+                                 TopapelLayerConfig)
+    step = (0.999 - 0.9) / max(lin_heads - 1, 1)
+    mixers = (ChunkAttentionConfig(heads, kv_heads, head, head ** -0.5, chunk, LinearRotConfig(500000.0, head, 4.0)),
+              MinGruConfig(gru),
+              LightningConfig(lin_heads, lin_dim, lin_dim, tuple(round(0.9 + step * h, 6) for h in range(lin_heads))))
+    return TopapelConfig(vocab=vocab, width=width, eps=1e-5, embedding_scale=width ** 0.5, logit_scale=1.0, logit_softcap=30.0,
+                         layers=tuple(TopapelLayerConfig(mixers[i % 3], ff) for i in range(layers)))
+
+
+# Topapel at the same two widths, depths, vocabularies, attention head shapes and feed-forward widths
+SHAPES.update({
+    "topapel-tiny": _topapel_shape(64, 512, 3, 4, 2, 16, 24, 80, 2, 32, 128),
+    "topapel-2k": _topapel_shape(2048, 32768, 8, 32, 8, 64, 1024, 2048, 16, 128, 8192),
+    "topapel-4k": _topapel_shape(4096, 32768, 4, 32, 8, 128, 1024, 4096, 32, 128, 14336),
+})
 DESIGN_PAIRS = (("zozosun-2k", "llama-2k"), ("zozosun-4k", "llama-4k"), ("timopel-2k", "llama-2k"),
                 ("timopel-4k", "llama-4k"), ("kotipel-2k", "llama-2k"), ("kotipel-4k", "llama-4k"),
-                ("robuvik-2k", "llama-2k"), ("robuvik-4k", "llama-4k"))
+                ("robuvik-2k", "llama-2k"), ("robuvik-4k", "llama-4k"), ("topapel-2k", "llama-2k"),
+                ("topapel-4k", "llama-4k"))
 
 
 def generate_requests(input_length: int, output_length: int, num_sequences: int, vocab_size: int,

@@ -749,7 +749,7 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
     const int full_hi = __builtin_amdgcn_readfirstlane((ctx_before + j_lo - 31) >> 5);
     const int full_lo = __builtin_amdgcn_readfirstlane((first_seen_key(ctx_before + j_hi, window, chunk) + 31) >> 5);
 
-    int qpos[NT], qlo[NT], tok[NT], head[NT];
+    int qpos[NT], tok[NT], head[NT];
     bool rvalid[NT];
     Frag qf[NT][DC];
     float m[NT], m_raw[NT];
@@ -764,7 +764,6 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
       tok[n] = q_begin + j;
       head[n] = hk * G + (rowc - j * G);
       qpos[n] = ctx_before + j;
-      qlo[n] = first_seen_key(qpos[n], window, chunk);
       const bf16_t* qp = q + (size_t)tok[n] * q_stride + (size_t)head[n] * HD;
 #pragma unroll
       for (int dc = 0; dc < DC; ++dc) {
@@ -815,6 +814,14 @@ __global__ __launch_bounds__(512) void prompt_attention_kernel(
       // some key of these blocks is invisible to some row: the causal edge, the window's edge, a
       // block beyond the tile's last key
       if (kb < full_lo || kb + KB - 1 > full_hi) {
+        // (the rows' first keys are made here, at the edges, and not kept: registers are short in this loop)
+        int qlo[NT];
+#pragma unroll
+        for (int n = 0; n < NT; ++n) {
+          int p = qpos[n];
+          asm volatile("" : "+v"(p));
+          qlo[n] = first_seen_key(p, window, chunk);
+        }
 #pragma unroll
         for (int h = 0; h < KB; ++h)
 #pragma unroll

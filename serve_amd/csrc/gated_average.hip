@@ -15,6 +15,7 @@
 
 #define GA_TILE 32
 #define GA_AHEAD 8          // tokens whose loads are in flight together
+#define GA_CHAIN 32         // tiles whose rows are read together on the way to a tile's first state
 
 // PMAX: upper bound of `parts`; the parts are loaded together, one beyond `parts` from a clamped address and dropped
 template <int PMAX>
@@ -116,16 +117,16 @@ __global__ __launch_bounds__(256) void gated_average_tile_kernel(
     // the tile begins inside a segment: the chain through the tiles before it, from the one in which the segment began
     int p = cu_q[seg] / GA_TILE;
     S = scratch[(size_t)p * 3 * W + W + c];
-    for (++p; p < tile; p += GA_AHEAD) {
-      float shrink[GA_AHEAD], add[GA_AHEAD];
+    for (++p; p < tile; p += GA_CHAIN) {
+      float shrink[GA_CHAIN], add[GA_CHAIN];
 #pragma unroll
-      for (int i = 0; i < GA_AHEAD; ++i) {
+      for (int i = 0; i < GA_CHAIN; ++i) {
         const float* r = scratch + (size_t)min(p + i, tile - 1) * 3 * W + c;
         shrink[i] = r[0];
         add[i] = r[W];
       }
 #pragma unroll
-      for (int i = 0; i < GA_AHEAD; ++i)
+      for (int i = 0; i < GA_CHAIN; ++i)
         if (p + i < tile) S = fmaf(shrink[i], S, add[i]);
     }
   }

@@ -11,6 +11,8 @@
 // The decays travel as their logarithms (<= 0), which is how both preparations get them and what a pass over several
 // tokens sums.  All arithmetic is fp32, also on the matrix cores (v_mfma_f32_16x16x4_f32); template types are the
 // storage of projections and outputs.
+#include <type_traits>
+
 #include "common.h"
 
 #define RS_MAX_TAPS 16
@@ -418,6 +420,236 @@ __global__ __launch_bounds__(256) void decay_scan_block_kernel(
 }
 
 // ---------------------------------------------------------------------------------------------
+// The same for one decay per head (and token), where the decays of a pass are numbers and not vectors over the channels:
+//
+//   o_t = e^(b_t) S0^T q_t  +  sum_(s<=t) e^(b_t - b_s) (q_t . k_s) v_s
+//   S   = e^(b_15) S0  +  sum_s k_s (e^(b_15 - b_s) v_s)^T
+//
+// q and k enter their products as they are, the decays multiply 16 x 16 scores, four rows of the read-out and four
+// values a lane.  Every lane of a wave's four rows of sixteen holds b_t of one token; the values come straight from
+// memory in the order the products want; q and k lie in LDS twice, so that a pass has one barrier before its products
+// and one between the two halves of the scores.  VEC: q and k in groups of four channels (dk, the strides and the
+// bases are multiples of four elements).
+// ---------------------------------------------------------------------------------------------
+__device__ __forceinline__ void read_four(const float* p, float (&f)[4]) {
+  const float4 v = *reinterpret_cast<const float4*>(p);
+  f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
+}
+template <typename TQ>
+struct Four;
+template <>
+struct Four<float> {
+  float4 v;
+  __device__ __forceinline__ void load(const float* p) { v = *reinterpret_cast<const float4*>(p); }
+  __device__ __forceinline__ void get(float (&f)[4]) const { f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w; }
+};
+template <>
+struct Four<bf16_t> {
+  uint2 v;
+  __device__ __forceinline__ void load(const bf16_t* p) { v = *reinterpret_cast<const uint2*>(p); }
+  __device__ __forceinline__ void get(float (&f)[4]) const {
+    f[0] = bf16_bits_to_float(v.x & 0xffffu);
+    f[1] = bf16_bits_to_float(v.x >> 16);
+    f[2] = bf16_bits_to_float(v.y & 0xffffu);
+    f[3] = bf16_bits_to_float(v.y >> 16);
+  }
+};
+
+template <typename TQ, int NT, bool VEC>
+__global__ __launch_bounds__(256) void decay_scan_head_kernel(
+    const TQ* __restrict__ q, const TQ* __restrict__ k, const TQ* __restrict__ v, long long q_stride,
+    long long k_stride, long long v_stride, const float* __restrict__ log_decay, long long decay_stride, int silu,
+    float q_scale, float* __restrict__ state, long long state_stride, const int* __restrict__ cu_q,
+    const int* __restrict__ state_slots, float* __restrict__ o, int H, int Hk, int dk, int dv, int RPT, int CPT,
+    int mode, int piece, int pieces, float* __restrict__ scratch, long long scratch_stride, long long scratch_decays) {
+  constexpr int DKP = 16 * NT;                   // the key channels, padded
+  constexpr int ST = DKP + 4;
+  constexpr int PER = VEC ? 4 : 1;               // channels of a load
+  constexpr int NL = VEC ? (NT + 3) / 4 : NT;    // loads of q, and of k, a thread
+  __shared__ __attribute__((aligned(16))) float sq[2][16][ST];
+  __shared__ __attribute__((aligned(16))) float sk[2][16][ST];
+  __shared__ float sap[4][16][17];
+  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, g = lane >> 4, j = lane & 15;
+  const int tile = blockIdx.x, h = blockIdx.y, seg = blockIdx.z / pieces, pj = blockIdx.z - seg * pieces;
+  const int hk = h / (H / Hk);
+  const int slot = state_slots[seg];
+  const int whole = cu_q[seg + 1] - cu_q[seg];   // the segment; this workgroup's piece of it: n tokens from t0
+  const int t0 = cu_q[seg] + pj * piece, n = min(piece, cu_q[seg + 1] - t0);
+  if (n <= 0) return;
+  const bool split = whole > piece;
+  if (mode == RS_PIECE_STATES && !split) return;
+  const int col = tile * 64 + w * 16 + j;        // this lane's column of S and o
+  const int seq_tiles = (dv + 16 * CPT - 1) / (16 * CPT);
+  auto state_at = [&](int row) -> size_t {       // where the token-by-token kernel keeps (row, col) of head h
+    return (((size_t)h * seq_tiles + col / (16 * CPT)) * RPT + row % RPT) * (size_t)(256 * CPT) +
+           (size_t)(((col / CPT) % 16) * 16 + row / RPT) * CPT + col % CPT;
+  };
+  int cut_before = 0;
+  if (split)
+    for (int s2 = 0; s2 < seg; ++s2) cut_before += (cu_q[s2 + 1] - cu_q[s2] > piece) ? 1 : 0;
+  float* const mine = scratch + (size_t)(cut_before * pieces + pj) * scratch_stride;
+  float* st = col >= dv ? nullptr : (split ? mine : (slot >= 0 ? state + (size_t)slot * state_stride : nullptr));
+  rs_f4 S[NT];
+#pragma unroll
+  for (int m = 0; m < NT; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) S[m][r] = (st && mode != RS_PIECE_STATES) ? st[state_at(16 * m + 4 * g + r)] : 0.f;
+  float btotal = 0.f;
+
+  // the inputs of a pass, in registers as they were loaded; places outside the segment or the head load a
+  // neighbour's value and are masked at use
+  float rla;
+  typename std::conditional<VEC, Four<TQ>, TQ>::type rq[NL], rk[NL];
+  TQ rv[4];
+  unsigned lo, qo[NL], ko[NL], vo[4];
+  auto place = [&](int last) {
+    lo = (unsigned)min(j, last) * (unsigned)decay_stride;
+#pragma unroll
+    for (int e = 0; e < NL; ++e) {
+      const int idx = (tid + 256 * e) * PER;
+      const unsigned tt = (unsigned)min(idx / DKP, last), cc = (unsigned)min(idx % DKP, dk - PER);
+      qo[e] = tt * (unsigned)q_stride + cc;
+      ko[e] = tt * (unsigned)k_stride + cc;
+    }
+#pragma unroll
+    for (int s4 = 0; s4 < 4; ++s4) vo[s4] = (unsigned)min(4 * s4 + g, last) * (unsigned)v_stride + (unsigned)min(col, dv - 1);
+  };
+  auto fetch = [&](int c0) {
+    const size_t tok = (size_t)(t0 + c0);
+    const TQ* qb = q + tok * q_stride + (size_t)hk * dk;
+    const TQ* kb = k + tok * k_stride + (size_t)hk * dk;
+    const TQ* vb = v + tok * v_stride + (size_t)h * dv;
+    rla = log_decay[tok * decay_stride + h + lo];
+#pragma unroll
+    for (int e = 0; e < NL; ++e) {
+      if constexpr (VEC) {
+        if (mode != RS_PIECE_STATES) rq[e].load(qb + qo[e]);
+        rk[e].load(kb + ko[e]);
+      } else {
+        if (mode != RS_PIECE_STATES) rq[e] = qb[qo[e]];
+        rk[e] = kb[ko[e]];
+      }
+    }
+#pragma unroll
+    for (int s4 = 0; s4 < 4; ++s4) rv[s4] = vb[vo[s4]];
+  };
+  place(min(16, n) - 1);
+  fetch(0);
+  for (int c0 = 0; c0 < n; c0 += 16) {
+    const int m = min(16, n - c0), buf = (c0 >> 4) & 1;
+    // b_t of token t = j, in every row of sixteen lanes
+    float b = j < m ? rla : 0.f;
+#pragma unroll
+    for (int x = 1; x < 16; x <<= 1) {
+      const float y = __shfl_up(b, x, 16);
+      if (j >= x) b += y;
+    }
+    const float b15 = __shfl(b, 15, 16);
+    btotal += b15;
+    float vc[4];
+#pragma unroll
+    for (int s4 = 0; s4 < 4; ++s4) vc[s4] = (4 * s4 + g < m && col < dv) ? read_qkv(rv[s4], silu) : 0.f;
+#pragma unroll
+    for (int e = 0; e < NL; ++e) {
+      const int idx = (tid + 256 * e) * PER, t = idx / DKP, c = idx % DKP;
+      if (VEC && NT < 4 && t > 15) break;        // (fewer groups than threads)
+      const bool in = t < m && c < dk;
+      if constexpr (VEC) {
+        float kf[4], qf[4];
+        rk[e].get(kf);
+        if (mode != RS_PIECE_STATES) rq[e].get(qf);
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+          kf[x] = in ? (silu ? short_silu(kf[x]) : kf[x]) : 0.f;
+          if (mode != RS_PIECE_STATES) qf[x] = in ? (silu ? short_silu(qf[x]) : qf[x]) * q_scale : 0.f;
+        }
+        *reinterpret_cast<float4*>(&sk[buf][t][c]) = make_float4(kf[0], kf[1], kf[2], kf[3]);
+        if (mode != RS_PIECE_STATES) *reinterpret_cast<float4*>(&sq[buf][t][c]) = make_float4(qf[0], qf[1], qf[2], qf[3]);
+      } else {
+        sk[buf][t][c] = in ? read_qkv(rk[e], silu) : 0.f;
+        if (mode != RS_PIECE_STATES) sq[buf][t][c] = in ? read_qkv(rq[e], silu) * q_scale : 0.f;
+      }
+    }
+    if (c0 + 16 < n) {                           // in flight while the products run
+      if (n - (c0 + 16) < 16) place(n - (c0 + 16) - 1);
+      fetch(c0 + 16);
+    }
+    float bs[4];
+#pragma unroll
+    for (int s4 = 0; s4 < 4; ++s4) bs[s4] = __shfl(b, 4 * s4 + g, 16);
+    __syncthreads();                             // q and k of the pass are there
+    if (mode != RS_PIECE_STATES) {
+      // each wave a quarter of the channels of the scores q_t . k_s
+      rs_f4 acc = {0.f, 0.f, 0.f, 0.f};
+      if (NT >= 4) {
+#pragma unroll
+        for (int i = 0; i < NT / 4; ++i) {
+          float qf[4], kf[4];
+          read_four(&sq[buf][j][w * 4 * NT + 16 * i + 4 * g], qf);
+          read_four(&sk[buf][j][w * 4 * NT + 16 * i + 4 * g], kf);
+#pragma unroll
+          for (int x = 0; x < 4; ++x) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[x], kf[x], acc, 0, 0, 0);
+        }
+      } else {
+#pragma unroll
+        for (int s4 = 0; s4 < NT; ++s4)
+          acc = __builtin_amdgcn_mfma_f32_16x16x4f32(sq[buf][j][w * 4 * NT + 4 * s4 + g], sk[buf][j][w * 4 * NT + 4 * s4 + g], acc, 0, 0, 0);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) sap[w][4 * g + r][j] = acc[r];
+      // the read-out of the state before the pass (two chains of products)
+      rs_f4 oc = {0.f, 0.f, 0.f, 0.f}, od = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int mt = 0; mt < NT; ++mt) {
+        float a4[4];
+        read_four(&sq[buf][j][16 * mt + 4 * g], a4);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          if (mt & 1) od = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[r], S[mt][r], od, 0, 0, 0);
+          else oc = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[r], S[mt][r], oc, 0, 0, 0);
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) oc[r] = (oc[r] + od[r]) * short_exp(__shfl(b, 4 * g + r, 16));
+      __syncthreads();                           // the scores' quarters are there
+      // this lane's scores: token j with tokens 4 s4 + g
+#pragma unroll
+      for (int s4 = 0; s4 < 4; ++s4) {
+        const int s = 4 * s4 + g;
+        const float dot = (sap[0][j][s] + sap[1][j][s]) + (sap[2][j][s] + sap[3][j][s]);
+        const float a = s <= j ? dot * short_exp(b - bs[s4]) : 0.f;
+        oc = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vc[s4], oc, 0, 0, 0);
+      }
+      if (col < dv) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (4 * g + r < m) o[((size_t)(t0 + c0 + 4 * g + r) * H + h) * dv + col] = oc[r];
+      }
+    }
+    // the state after the pass
+    const float shrink = short_exp(b15);
+#pragma unroll
+    for (int s4 = 0; s4 < 4; ++s4) vc[s4] *= short_exp(b15 - bs[s4]);
+#pragma unroll
+    for (int mt = 0; mt < NT; ++mt) {
+      rs_f4 sm = S[mt];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) sm[r] *= shrink;
+#pragma unroll
+      for (int s4 = 0; s4 < 4; ++s4) sm = __builtin_amdgcn_mfma_f32_16x16x4f32(sk[buf][4 * s4 + g][16 * mt + j], vc[s4], sm, 0, 0, 0);
+      S[mt] = sm;
+    }
+  }
+  if (st && (mode == RS_PIECE_STATES || !split)) {
+#pragma unroll
+    for (int m = 0; m < NT; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) st[state_at(16 * m + 4 * g + r)] = S[m][r];
+  }
+  if (mode == RS_PIECE_STATES && tile == 0 && tid < DKP) mine[scratch_decays + (size_t)h * DKP + tid] = short_exp(btotal);
+}
+
+// ---------------------------------------------------------------------------------------------
 // Between the two passes over the pieces of long segments: from the request's state (or zeros) S, piece after piece,
 // the piece's row takes S, the state it starts from, and S <- D S + (what the piece's tokens add), D the piece's
 // decay of the row's key channel; the state after the last piece goes to the request.  A thread per float of a
@@ -442,11 +674,22 @@ __global__ __launch_bounds__(256) void decay_scan_chain_kernel(float* __restrict
   const int h = hi / (tiles * RPT), row = (thread & 15) * RPT + hi % RPT;
   const int slot = state_slots[seg];
   float S = slot >= 0 ? state[(size_t)slot * state_stride + at] : 0.f;
-  for (int pj = 0; pj < count; ++pj) {
-    float* mine = scratch + (size_t)(cut_before * pieces + pj) * scratch_stride;
-    const float add = mine[at], D = mine[scratch_decays + (size_t)h * DKP + row];
-    mine[at] = S;
-    S = fmaf(D, S, add);
+  float* first = scratch + (size_t)(cut_before * pieces) * scratch_stride;
+  constexpr int AHEAD = 8;                       // pieces whose rows are read together
+  for (int pj = 0; pj < count; pj += AHEAD) {
+    float add[AHEAD], D[AHEAD];
+#pragma unroll
+    for (int x = 0; x < AHEAD; ++x) {
+      const float* mine = first + (size_t)min(pj + x, count - 1) * scratch_stride;
+      add[x] = mine[at];
+      D[x] = mine[scratch_decays + (size_t)h * DKP + row];
+    }
+#pragma unroll
+    for (int x = 0; x < AHEAD; ++x) {
+      if (pj + x >= count) break;
+      first[(size_t)(pj + x) * scratch_stride + at] = S;
+      S = fmaf(D[x], S, add[x]);
+    }
   }
   if (slot >= 0) state[(size_t)slot * state_stride + at] = S;
 }
@@ -458,6 +701,26 @@ static int launch_scan_block(int rpt, int cpt, const void* q, const void* k, con
                              int dk, int dv, int mode, int piece, int pieces, float* scratch, long long scratch_stride,
                              long long scratch_decays, hipStream_t stream) {
   dim3 grid((dv + 63) / 64, H, B * pieces), block(256);
+  if (!per_channel) {
+    const bool vec = dk % 4 == 0 && qs % 4 == 0 && ks % 4 == 0 &&
+                     !(((uintptr_t)q | (uintptr_t)k) & (4 * sizeof(TQ) - 1));
+#define GOV(N, V) hipLaunchKernelGGL((decay_scan_head_kernel<TQ, N, V>), grid, block, 0, stream, (const TQ*)q, (const TQ*)k, (const TQ*)v, qs, ks, vs, decay, decay_stride, silu, q_scale, state, state_stride, cu_q, slots, o, H, Hk, dk, dv, rpt, cpt, mode, piece, pieces, scratch, scratch_stride, scratch_decays)
+#define GO(N)          \
+  do {                 \
+    if (vec) GOV(N, true); \
+    else GOV(N, false); \
+  } while (0)
+    switch (rpt) {
+      case 1: GO(1); break;
+      case 2: GO(2); break;
+      case 4: GO(4); break;
+      case 8: GO(8); break;
+      default: return SA_ERR_UNSUPPORTED;
+    }
+#undef GO
+#undef GOV
+    return 0;
+  }
 #define GO(N) hipLaunchKernelGGL((decay_scan_block_kernel<TQ, N>), grid, block, 0, stream, (const TQ*)q, (const TQ*)k, (const TQ*)v, qs, ks, vs, decay, per_channel, decay_stride, silu, q_scale, state, state_stride, cu_q, slots, o, H, Hk, dk, dv, rpt, cpt, mode, piece, pieces, scratch, scratch_stride, scratch_decays)
   switch (rpt) {
     case 1: GO(1); break;
@@ -493,7 +756,7 @@ extern "C" int sa_decay_scan(const void* q, const void* k, const void* v, int dt
   const int rpt = scan_rpt(dk), cpt = scan_cpt(dv);
   const long long far_stride = 1LL << 27;         // the passes over sixteen tokens keep 32-bit offsets within a pass
   if (max_q >= RS_BLOCK_MIN_TOKENS && dk <= RS_BLOCK_MAX_DK && (dtype == SA_F32 || dtype == SA_BF16) &&
-      q_stride < far_stride && k_stride < far_stride && v_stride < far_stride && (long long)H * dk < far_stride) {
+      q_stride < far_stride && k_stride < far_stride && v_stride < far_stride && (long long)H * dk < far_stride && decay_stride < far_stride) {
     // piece > 0: segments longer than `piece` tokens (a multiple of 16) run as pieces side by side; scratch: fp32 rows
     // of scratch_stride >= state floats + H 16 rpt floats, ceil(max_q / piece) for every segment that is cut, zeroed
     const long long floats = sa_decay_scan_state_floats(H, dk, dv);
@@ -824,6 +1087,78 @@ __global__ __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) void gated_group_nor
   }
 }
 
+// The same for groups that are multiples of four and at most 8,192 long, from aligned rows: 16-byte vectors, one workgroup a
+// group (256 threads, NG groups of four each), every load of a group issued before anything is computed.
+__device__ __forceinline__ float4 rs_ld4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 rs_ld4(const bf16_t* p) {
+  const uint2 u = *reinterpret_cast<const uint2*>(p);
+  return make_float4(bf16_bits_to_float(u.x & 0xffffu), bf16_bits_to_float(u.x >> 16),
+                     bf16_bits_to_float(u.y & 0xffffu), bf16_bits_to_float(u.y >> 16));
+}
+__device__ __forceinline__ void rs_st4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+__device__ __forceinline__ void rs_st4(bf16_t* p, float4 v) {
+  uint2 u;
+  u.x = (uint32_t)float_to_bf16_bits(v.x) | ((uint32_t)float_to_bf16_bits(v.y) << 16);
+  u.y = (uint32_t)float_to_bf16_bits(v.z) | ((uint32_t)float_to_bf16_bits(v.w) << 16);
+  *reinterpret_cast<uint2*>(p) = u;
+}
+
+template <typename TA, int NG, bool SKIP>
+__global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(
+    const float* __restrict__ o, const float* __restrict__ skip_x, long long skip_stride,
+    const float* __restrict__ skip_d, int dv, const TA* __restrict__ gate, long long gate_stride, int gate_col,
+    const float* __restrict__ w, int wn, int group, int gate_first, int gate_kind, float eps, TA* __restrict__ y, int n) {
+  __shared__ float scratch[16];
+  const int groups = n / group;
+  const int t = blockIdx.x / groups, i0 = (blockIdx.x - t * groups) * group;
+  const float* orow = o + (size_t)t * n + i0;
+  const TA* grow = gate + (size_t)t * gate_stride + gate_col + i0;
+  const int quads = group >> 2;
+  float4 u[NG], gt[NG], wv[NG];
+#pragma unroll
+  for (int x = 0; x < NG; ++x) {
+    const int i = min((int)threadIdx.x + x * 256, quads - 1) * 4;
+    u[x] = rs_ld4(orow + i);
+    gt[x] = rs_ld4(grow + i);
+    wv[x] = rs_ld4(w + (i0 + i) % wn);
+    if (SKIP) {
+      const float4 s4 = rs_ld4(skip_x + (size_t)t * skip_stride + i0 + i);
+      const float d = skip_d[(i0 + i) / dv];
+      u[x].x = fmaf(d, s4.x, u[x].x);
+      u[x].y = fmaf(d, s4.y, u[x].y);
+      u[x].z = fmaf(d, s4.z, u[x].z);
+      u[x].w = fmaf(d, s4.w, u[x].w);
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int x = 0; x < NG; ++x) {
+    gt[x].x = readout_gate(gt[x].x, gate_kind);
+    gt[x].y = readout_gate(gt[x].y, gate_kind);
+    gt[x].z = readout_gate(gt[x].z, gate_kind);
+    gt[x].w = readout_gate(gt[x].w, gate_kind);
+    if (gate_first) {
+      u[x].x *= gt[x].x;
+      u[x].y *= gt[x].y;
+      u[x].z *= gt[x].z;
+      u[x].w *= gt[x].w;
+    }
+    const float in = (int)threadIdx.x + x * 256 < quads ? 1.f : 0.f;
+    ss += in * (u[x].x * u[x].x + u[x].y * u[x].y + u[x].z * u[x].z + u[x].w * u[x].w);
+  }
+  ss = block_sum(ss, scratch);
+  const float rs = 1.0f / sqrtf(ss / (float)group + eps);
+#pragma unroll
+  for (int x = 0; x < NG; ++x) {
+    const int qd = threadIdx.x + x * 256;
+    if (qd < quads) {
+      float4 r = make_float4((u[x].x * rs) * wv[x].x, (u[x].y * rs) * wv[x].y, (u[x].z * rs) * wv[x].z, (u[x].w * rs) * wv[x].w);
+      if (!gate_first) r = make_float4(r.x * gt[x].x, r.y * gt[x].y, r.z * gt[x].z, r.w * gt[x].w);
+      rs_st4(y + (size_t)t * n + i0 + qd * 4, r);
+    }
+  }
+}
+
 extern "C" int sa_gated_group_norm(const float* o, const float* skip_x, long long skip_stride, const float* skip_d,
                                    int dv, const void* gate, int dtype, long long gate_stride, int gate_col,
                                    const float* w, int wn, int group, int gate_first, int gate_kind, float eps, void* y, int T, int n,
@@ -833,6 +1168,34 @@ extern "C" int sa_gated_group_norm(const float* o, const float* skip_x, long lon
       gate_kind > 1)
     return SA_ERR_ARG;
   const long long units = (long long)T * (n / group);
+  const int esize = dtype == SA_F32 ? 4 : 2;
+  const bool vec = group % 4 == 0 && group >= 512 && group <= 8192 && wn % 4 == 0 && gate_stride % 4 == 0 && gate_col % 4 == 0 &&
+                   !(((uintptr_t)o | (uintptr_t)w | (uintptr_t)skip_x) & 15) && !(((uintptr_t)gate | (uintptr_t)y) & (4 * esize - 1)) &&
+                   (!skip_x || (skip_stride % 4 == 0 && dv % 4 == 0)) && units <= 0x7fffffffLL &&
+                   (dtype == SA_F32 || dtype == SA_BF16);
+  if (vec) {
+    const int ng = (group / 4 + 255) / 256;
+#define GOV(TA, NG, SK) hipLaunchKernelGGL((gated_group_norm_vec_kernel<TA, NG, SK>), dim3((unsigned)units), dim3(256), 0, stream, o, skip_x, skip_stride, skip_d, dv, (const TA*)gate, gate_stride, gate_col, w, wn, group, gate_first, gate_kind, eps, (TA*)y, n)
+#define GOS(TA, NG)              \
+  do {                           \
+    if (skip_x) GOV(TA, NG, true); \
+    else GOV(TA, NG, false);     \
+  } while (0)
+#define GON(TA)                  \
+  do {                           \
+    if (ng <= 1) GOS(TA, 1);     \
+    else if (ng <= 2) GOS(TA, 2); \
+    else if (ng <= 4) GOS(TA, 4); \
+    else GOS(TA, 8);             \
+  } while (0)
+    if (dtype == SA_F32) GON(float);
+    else GON(bf16_t);
+#undef GON
+#undef GOS
+#undef GOV
+    SA_LAUNCH_CHECK();
+    return 0;
+  }
   const bool whole = group >= 1024;             // a workgroup a group
   const long long blocks = whole ? units : (units + 3) / 4;
   if (blocks > 0x7fffffffLL) return SA_ERR_ARG;

@@ -974,7 +974,9 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
         rows = cut * -(-max_q // piece)
         row = need + heads * 16 * _pow2_rows(dk)
         if max_q > piece and cut > 0 and rows * row * 4 <= SCAN_PIECE_SCRATCH_BYTES:
-            scratch = torch.zeros((rows, row), dtype=torch.float32, device=out.device)
+            # (zeros where columns of the state are padding that nobody writes)
+            make = torch.empty if dv % 64 == 0 else torch.zeros
+            scratch = make((rows, row), dtype=torch.float32, device=out.device)
         else:
             piece = 0
     _ret(lib.sa_decay_scan(_ptr(q), _ptr(k), _ptr(v), c_int(_code(q)), LL(q.stride(0)), LL(k.stride(0)), LL(v.stride(0)),
