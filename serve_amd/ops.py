@@ -1095,7 +1095,7 @@ def gated_group_norm(o: torch.Tensor, gate_rows: torch.Tensor, gate_col: int, we
 # element-wise gated averages S_t = (1 - z_t) S_(t-1) + z_t c_t
 # ---------------------------------------------------------------------------------------------
 GATED_AVERAGE_TILE = 32          # tokens a workgroup takes (csrc/gated_average.hip: GA_TILE)
-GATED_AVERAGE_SHORT = 16         # steps whose longest segment has at most this many tokens go segment by segment
+GATED_AVERAGE_SHORT = 16         # segments of at most this many tokens go one by one (GA_SHORT)
 
 
 def gated_average(rows: torch.Tensor, bias: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor) -> torch.Tensor:
@@ -1117,14 +1117,17 @@ def gated_average(rows: torch.Tensor, bias: torch.Tensor, state: torch.Tensor, c
     _i32(ctx.state_slots, B, "state_slots")
     lib = load_library("gated_average")
     max_q = int(getattr(ctx, "max_q_len", 0) or T)
-    by_segment = max_q <= GATED_AVERAGE_SHORT
+    any_long = max_q > GATED_AVERAGE_SHORT
+    any_short = B > 1 or not any_long             # (a single segment is one or the other; a bound cannot rule short ones out)
+    if B == 1 and max_q != T:
+        any_short = any_long = True               # (a step replayed from a graph: its one segment may have any length)
     scratch = None
-    if not by_segment and T > GATED_AVERAGE_TILE:
+    if any_long and T > GATED_AVERAGE_TILE:
         scratch = torch.empty((-(-T // GATED_AVERAGE_TILE), 3 * W), dtype=torch.float32, device=out.device)
     _ret(lib.sa_gated_average(_ptr(rows), c_int(parts), _ptr(bias), _ptr(state), ctypes.c_longlong(state.stride(0)),
                               _ptr(ctx.cu_q), _ptr(ctx.seg_of_token), _ptr(ctx.state_slots), _ptr(out), c_int(_code(out)),
-                              _ptr(scratch), c_int(T), c_int(B), c_int(W), c_int(1 if by_segment else 0), _stream()),
-         "gated_average")
+                              _ptr(scratch), c_int(T), c_int(B), c_int(W), c_int(1 if any_short else 0),
+                              c_int(1 if any_long else 0), _stream()), "gated_average")
     return out
 
 
