@@ -118,6 +118,17 @@ def test_parts_refuse_what_they_do_not_compute():
         Model(type(spec)(**{**spec.__dict__, "layers": [parallel], "run_order": spec.run_order[:1]}))
 
 
+def test_random_model_from_the_command_line(tmp_path):
+    """`random-model` writes a folder for the named shape, which the plain model can run."""
+    from serve_amd.__main__ import main
+    folder = str(tmp_path / "a")
+    assert main(["random-model", "--shape", "topapel-tiny", "--out", folder, "--seed", "5"]) == 0
+    cfg = tm.plain_config(folder)
+    assert TopapelConfig.from_hf_dict(cfg).to_hf_dict() == cfg
+    logits = tm.plain_logits(folder, [1, 2, 3, 4, 5])
+    assert logits.shape == (5, 512) and torch.isfinite(logits).all() and logits.abs().max() <= cfg["logit_softcap"]
+
+
 # -- retention by chunks --------------------------------------------------------------------------------
 def test_retention_rules():
     assert [first_seen(Chunks(5), p) for p in (0, 4, 5, 9, 10, 23)] == [0, 0, 5, 5, 10, 20]
