@@ -371,7 +371,7 @@ def step_of(lens, slots=None, ctx_lens=None):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("H,G,D,page,chunk", [(4, 2, 32, 4, 10), (6, 2, 96, 16, 64), (3, 1, 16, 12, 33), (8, 1, 128, 32, 100), (2, 2, 136, 8, 40),
+@pytest.mark.parametrize("H,G,D,page,chunk", [(4, 2, 32, 4, 10), (9, 3, 80, 16, 72), (3, 1, 16, 12, 33), (8, 1, 128, 32, 100), (2, 2, 136, 8, 40),
                                               (20, 1, 64, 16, 48), (2, 1, 64, 16, 1), (4, 4, 48, 16, 4096)])
 def test_attention_in_chunks(dtype, H, G, D, page, chunk):
     """Every attention kernel (a wave a row; tiles and single tokens in float32; one wave, one workgroup and prompt
@@ -435,7 +435,7 @@ def test_attention_in_chunks(dtype, H, G, D, page, chunk):
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H,G,D,Dp,rot,shared,T", [
-    (4, 2, 32, 32, 16, True, 11), (6, 2, 96, 96, 96, True, 40), (3, 3, 10, 16, 4, True, 11), (2, 1, 136, 144, 64, True, 11),
+    (4, 2, 32, 32, 16, True, 11), (9, 3, 80, 80, 80, True, 40), (3, 3, 10, 16, 4, True, 11), (2, 1, 136, 144, 64, True, 11),
     (5, 1, 24, 32, 24, True, 33), (4, 4, 16, 16, 0, True, 11), (3, 1, 64, 64, 32, False, 70), (2, 2, 20, 32, 6, False, 11),
     (8, 2, 128, 128, 128, True, 300), (2, 1, 8, 16, 2, True, 11)])
 def test_norm_rotation_and_cache_write(dtype, H, G, D, Dp, rot, shared, T):
@@ -524,15 +524,15 @@ def test_polynomial_of_normed_powers(dtype, T, n, parts):
 def test_scaled_and_capped_logits():
     from serve_amd import ops
     g = torch.Generator().manual_seed(4)
-    for R, V in ((1, 5), (3, 641), (2, 40000)):
+    for R, V in ((1, 5), (3, 513), (2, 40000)):
         y = 30.0 * torch.randn(R, V, generator=g)
-        got = ops.scale_soft_cap(y.cuda(), 0.5, 15.0).double().cpu()
-        assert torch.allclose(got, tp.soft_cap(0.5 * y.double(), 15.0), atol=1e-5, rtol=1e-5)
+        got = ops.scale_soft_cap(y.cuda(), 0.4, 12.0).double().cpu()
+        assert torch.allclose(got, tp.soft_cap(0.4 * y.double(), 12.0), atol=1e-5, rtol=1e-5)
         assert torch.allclose(ops.scale_soft_cap(y.cuda(), 0.25, 0.0).cpu(), 0.25 * y)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("H,dk,dv", [(2, 16, 72), (3, 24, 40), (4, 128, 128), (2, 136, 24), (1, 1, 1), (6, 64, 32)])
+@pytest.mark.parametrize("H,dk,dv", [(2, 16, 72), (3, 24, 40), (4, 128, 128), (2, 136, 24), (1, 1, 1), (6, 48, 32)])
 @pytest.mark.parametrize("lens", [[1, 1, 1], [3, 1, 5], [40, 1, 2, 17], [700], [16, 300, 1, 1]])
 def test_recurrence_with_one_decay_a_head(dtype, H, dk, dv, lens):
     """Constant decays and z sigmoid(z) on q, k and v, over two steps of the same requests (short and long segments, long
