@@ -53,6 +53,10 @@ class RunEntry:
     pass_vector: Optional[int] = None
     # with a pass vector: the embedding's output (the stream as it was before the first layer) is added as well
     adds_embedding: bool = False
+    # another cache layer whose pages the mixer reads, where it keeps nothing per token itself: `cache` is then a layer of
+    # its own that holds at most its per-request state (where it has no state either, naming the other layer as `cache`
+    # without `writes_cache` does)
+    reads_pages_of: Optional[int] = None
 
 
 @dataclass(frozen=True)

@@ -52,6 +52,8 @@ SOURCES: Dict[str, str] = {
     "recurrent_scan": "recurrent_scan.hip",
     "gated_average": "gated_average.hip",
     "stream_ops": "stream_ops.hip",
+    "stream_mix": "stream_mix.hip",
+    "conv_attention": "conv_attention.hip",
 }
 # what a library is linked with beside the HIP runtime
 LINK: Dict[str, List[str]] = {"blaslt.hip": ["-lhipblaslt"]}

@@ -1,9 +1,14 @@
 // Routed experts: every token takes the `top` experts with the largest router logits, weighted by the
 // softmax over those logits alone (or: by their shares of the softmax over all experts, divided by the sum
-// of the chosen shares + 1e-20; or: by the sigmoid of each chosen logit as it is; each times a constant); an expert
+// of the chosen shares + 1e-20, chosen by shares plus a stored correction where there is one; or: by the sigmoid of each
+// chosen logit as it is; each times a constant); an expert
 // is down(gate(gate x, up x)) with one of the gates of common.h (silu(g) u and others).  The weight multiplies the
 // expert's output (in `combine`), or, where a design says so, its input: gate and up are linear in x, so
 // expert(w x) = down(gate(w gate x, w up x)), and the weight enters where the gate is applied.
+//
+// The router may have more outputs than there are experts: those behind the E experts are identity experts, whose output
+// is the token itself.  They are chosen and weighted like the others, but their rows are in no expert's list, and what
+// adds up a token's experts takes the token's own row for them.
 //
 // Nothing is read back to the host: the tokens are grouped by expert on the device, and the
 // products run over a list of (expert, rows) tiles that is built there, from a grid sized for
@@ -30,21 +35,63 @@
 // mode 1: the weights are shares of the softmax over all E logits, renormalised over the chosen ones
 // (p_k / S) / (sum_chosen p / S + 1e-20) with S the sum over all; mode 0: p_k / sum_chosen p; mode 2: the sigmoid of
 // every chosen logit, not normalised.  All times wscale.
+// corr (mode 1 only, or null): per output a number that is added to the share where the outputs are chosen, and not where
+// they are weighted.  E: all of the router's outputs.
 __device__ __forceinline__ void route_token(const float* __restrict__ z, int* __restrict__ ids, float* __restrict__ wts,
-                                            int E, int top, int lane, int mode, float wscale);
+                                            int E, int top, int lane, int mode, float wscale,
+                                            const float* __restrict__ corr);
 
 __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int ldz, int* __restrict__ ids,
                                                         float* __restrict__ wts, int T, int E, int top, int over_all,
-                                                        float wscale) {
+                                                        float wscale, const float* __restrict__ corr) {
   const int t = blockIdx.x * (blockDim.x / SA_WAVE) + threadIdx.x / SA_WAVE;
   if (t >= T) return;
   route_token(logits + (size_t)t * ldz, ids + (size_t)t * top, wts + (size_t)t * top, E, top,
-              threadIdx.x & (SA_WAVE - 1), over_all, wscale);
+              threadIdx.x & (SA_WAVE - 1), over_all, wscale, corr);
 }
 
 __device__ __forceinline__ void route_token(const float* __restrict__ z, int* __restrict__ ids, float* __restrict__ wts,
-                                            int E, int top, int lane, int mode, float wscale) {
+                                            int E, int top, int lane, int mode, float wscale,
+                                            const float* __restrict__ corr) {
   const int over_all = mode == 1;
+  if (corr) {
+    // shares of the softmax first: what is chosen is their sum with the correction
+    float big = -INFINITY;
+    for (int e = lane; e < E; e += SA_WAVE) big = fmaxf(big, z[e]);
+    big = wave_max(big);
+    float part = 0.f;
+    for (int e = lane; e < E; e += SA_WAVE) part += expf(z[e] - big);
+    const float all = wave_sum(part);
+    float pv = INFINITY, chosen = 0.f;
+    int pi = -1;
+    for (int k = 0; k < top; ++k) {
+      float bv = -INFINITY;
+      int bi = 0x7fffffff;
+      for (int e = lane; e < E; e += SA_WAVE) {
+        const float v = expf(z[e] - big) / all + corr[e];
+        const bool after = v < pv || (v == pv && e > pi);
+        if (after && (v > bv || (v == bv && e < bi))) { bv = v; bi = e; }
+      }
+#pragma unroll
+      for (int o = SA_WAVE / 2; o > 0; o >>= 1) {
+        const float ov = __shfl_xor(bv, o, SA_WAVE);
+        const int oi = __shfl_xor(bi, o, SA_WAVE);
+        if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+      }
+      bi = min(bi, E - 1);               // (logits that are no numbers choose nothing: stay within the table)
+      const float p = expf(z[bi] - big) / all;
+      chosen += p;
+      if (lane == 0) {
+        ids[k] = bi;
+        wts[k] = p;
+      }
+      pv = bv;
+      pi = bi;
+    }
+    if (lane == 0)
+      for (int k = 0; k < top; ++k) wts[k] = (wts[k] / (chosen + 1e-20f)) * wscale;
+    return;
+  }
   float prev_v = INFINITY;
   int prev_i = -1;
   float first = 0.f, sum = 0.f;
@@ -100,7 +147,8 @@ __device__ __forceinline__ void route_token(const float* __restrict__ z, int* __
 __device__ __forceinline__ void group_rows(const int* ids, int n, int E, int tile_rows, int* __restrict__ offsets,
                                            int* cursor, int* __restrict__ perm, int* __restrict__ tile_expert,
                                            int* __restrict__ tile_row0, int* __restrict__ num_tiles) {
-  for (int i = threadIdx.x; i < n; i += blockDim.x) atomicAdd(&cursor[ids[i]], 1);
+  for (int i = threadIdx.x; i < n; i += blockDim.x)
+    if (ids[i] < E) atomicAdd(&cursor[ids[i]], 1);          // (identity experts' rows are in no list)
   __syncthreads();
   if (threadIdx.x == 0) {
     int run = 0, tiles = 0;
@@ -119,7 +167,8 @@ __device__ __forceinline__ void group_rows(const int* ids, int n, int E, int til
     *num_tiles = tiles;
   }
   __syncthreads();
-  for (int i = threadIdx.x; i < n; i += blockDim.x) perm[atomicAdd(&cursor[ids[i]], 1)] = i;
+  for (int i = threadIdx.x; i < n; i += blockDim.x)
+    if (ids[i] < E) perm[atomicAdd(&cursor[ids[i]], 1)] = i;
 }
 
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int* ids, int n, int E, int tile_rows,
@@ -127,7 +176,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* ids, int n, 
                                                          int* __restrict__ perm, int* __restrict__ tile_expert,
                                                          int* __restrict__ tile_row0, int* __restrict__ num_tiles,
                                                          const float* __restrict__ logits, int ldz, int* ids_out,
-                                                         float* __restrict__ wts, int top, int over_all, float wscale) {
+                                                         float* __restrict__ wts, int top, int over_all, float wscale,
+                                                         const float* __restrict__ corr, int outputs) {
   __shared__ int lds_cursor[MOE_LDS_EXPERTS];
   const bool in_lds = E <= MOE_LDS_EXPERTS;              // (the counters are scratch: nobody reads them afterwards)
   for (int e = threadIdx.x; e < E; e += blockDim.x) {
@@ -138,8 +188,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* ids, int n, 
     // a step of few tokens: the routing is done here, a wave a token in turn, and saves a kernel
     const int waves = blockDim.x / SA_WAVE, T = n / top;
     for (int t = threadIdx.x / SA_WAVE; t < T; t += waves)
-      route_token(logits + (size_t)t * ldz, ids_out + (size_t)t * top, wts + (size_t)t * top, E, top,
-                  threadIdx.x & (SA_WAVE - 1), over_all, wscale);
+      route_token(logits + (size_t)t * ldz, ids_out + (size_t)t * top, wts + (size_t)t * top, outputs, top,
+                  threadIdx.x & (SA_WAVE - 1), over_all, wscale, corr);
   }
   __syncthreads();
   if (in_lds) group_rows(ids, n, E, tile_rows, offsets, lds_cursor, perm, tile_expert, tile_row0, num_tiles);
@@ -396,7 +446,7 @@ __global__ __launch_bounds__(256) void moe_mfma_kernel(const bf16_t* __restrict_
   }
 }
 
-// combine: grid (T, parts of a row).  shared: [parts, T, d] (TS), or null; sg: logits fp32, row stride ldz (null: no gate);
+// combine: grid (T, parts of a row).  ids (null: no identity experts): an id >= E takes row t of `own` [T, d].  shared: [parts, T, d] (TS), or null; sg: logits fp32, row stride ldz (null: no gate);
 // wts null: the rows are added as they are (their weights went into the experts' inputs).
 // TOPMAX / PMAX: upper bounds of `top` / `parts` (0: any number, in a loop): with bounds, all loads of an output
 // are issued before anything is added (rows beyond the bounds are read from a clamped place and dropped).
@@ -404,8 +454,16 @@ template <typename TS, int TOPMAX, int PMAX>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ yk, const float* __restrict__ wts,
                                                           const TS* __restrict__ shared, int parts, size_t part_stride,
                                                           const float* __restrict__ sg, int ldz, float* __restrict__ y,
-                                                          int top, int d) {
+                                                          int top, int d, const int* __restrict__ ids, int E,
+                                                          const void* __restrict__ own, int own_bf16) {
   const int t = blockIdx.x;
+  auto row_at = [&](int k, int i) -> float {
+    if (ids && ids[(size_t)t * top + k] >= E) {             // an identity expert: its row of yk holds nothing
+      const size_t at = (size_t)t * d + i;
+      return own_bf16 ? to_float(reinterpret_cast<const bf16_t*>(own)[at]) : reinterpret_cast<const float*>(own)[at];
+    }
+    return yk[((size_t)t * top + k) * d + i];
+  };
   float gate = 1.f;
   if (shared && sg) gate = 1.f / (1.f + expf(-sg[(size_t)t * ldz]));
   if (TOPMAX > 0) {
@@ -415,7 +473,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
     for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < d; i += blockDim.x * gridDim.y) {
       float a[TOPMAX > 0 ? TOPMAX : 1], sp[PMAX];
 #pragma unroll
-      for (int k = 0; k < TOPMAX; ++k) a[k] = yk[((size_t)t * top + min(k, top - 1)) * d + i];
+      for (int k = 0; k < TOPMAX; ++k) a[k] = row_at(min(k, top - 1), i);
 #pragma unroll
       for (int p = 0; p < PMAX; ++p) sp[p] = shared ? to_float(shared[min(p, parts - 1) * part_stride + (size_t)t * d + i]) : 0.f;
       float v = 0.f;
@@ -430,7 +488,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
   }
   for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < d; i += blockDim.x * gridDim.y) {
     float v = 0.f;
-    for (int k = 0; k < top; ++k) v += (wts ? wts[(size_t)t * top + k] : 1.f) * yk[((size_t)t * top + k) * d + i];
+    for (int k = 0; k < top; ++k) v += (wts ? wts[(size_t)t * top + k] : 1.f) * row_at(k, i);
     if (shared) {
       float sh = 0.f;
       for (int p = 0; p < parts; ++p) sh += to_float(shared[p * part_stride + (size_t)t * d + i]);
@@ -444,11 +502,11 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
 extern "C" int sa_moe_max_tiles(int rows, int E) { return (rows + 15) / 16 + E; }
 
 extern "C" int sa_moe_route(const float* logits, int ldz, int* ids, float* wts, int T, int E, int top,
-                            int over_all, float wscale, hipStream_t stream) {
+                            int over_all, float wscale, const float* corr, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (E <= 0 || top <= 0 || top > E || ldz < E) return SA_ERR_ARG;
+  if (E <= 0 || top <= 0 || top > E || ldz < E || (corr && over_all != 1)) return SA_ERR_ARG;
   dim3 grid((T + 3) / 4), block(256);
-  hipLaunchKernelGGL(moe_route_kernel, grid, block, 0, stream, logits, ldz, ids, wts, T, E, top, over_all, wscale);
+  hipLaunchKernelGGL(moe_route_kernel, grid, block, 0, stream, logits, ldz, ids, wts, T, E, top, over_all, wscale, corr);
   SA_LAUNCH_CHECK();
   return 0;
 }
@@ -459,7 +517,7 @@ extern "C" int sa_moe_route(const float* logits, int ldz, int* ids, float* wts, 
 #define MOE_SMALL_ROWS 1024
 
 // logits != nullptr (and T <= MOE_ROUTE_INSIDE): ids and wts are made here from the router's logits fp32 [T, ldz]
-// (over_all: the mode of route_token, 0 to 2).  in_wts (fp32 [T top], may be wts itself): the weights multiply the experts' inputs
+// (over_all: the mode of route_token, 0 to 2; corr and outputs: its correction and all of its outputs, at least E).  in_wts (fp32 [T top], may be wts itself): the weights multiply the experts' inputs
 #define MOE_ROUTE_INSIDE 16
 
 extern "C" int sa_moe_route_inside_limit() { return MOE_ROUTE_INSIDE; }
@@ -467,7 +525,7 @@ extern "C" int sa_moe_route_inside_limit() { return MOE_ROUTE_INSIDE; }
 extern "C" int sa_moe_experts(const void* h, int act_dtype, int* ids, const void* Wg, const void* Wu,
                               const void* Wd, int* ints, void* act, float* yk, int T, int top, int E, int d, int F,
                               const float* logits, int ldz, float* wts, int over_all, float wscale, int gate_kind,
-                              float gate_limit, const float* in_wts, hipStream_t stream) {
+                              float gate_limit, const float* in_wts, const float* corr, int outputs, hipStream_t stream) {
   if (T <= 0) return 0;
   const long long n = (long long)T * top;
   if (E <= 0 || top <= 0 || d <= 0 || F <= 0 || n > 0x3fffffffLL) return SA_ERR_ARG;
@@ -483,9 +541,10 @@ extern "C" int sa_moe_experts(const void* h, int act_dtype, int* ids, const void
   const bool small = n <= MOE_SMALL_ROWS;
   const int tile_rows = mfma ? (small ? 16 : 64) : MOE_TM;
   const int tiles = (int)((n + tile_rows - 1) / tile_rows) + E;
-  if (logits && (T > MOE_ROUTE_INSIDE || !wts || ldz < E || top > E)) return SA_ERR_ARG;
+  if (logits && (T > MOE_ROUTE_INSIDE || !wts || outputs < E || ldz < outputs || top > outputs || (corr && over_all != 1)))
+    return SA_ERR_ARG;
   hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, stream, ids, (int)n, E, tile_rows, offsets, cursor, perm,
-                     tile_expert, tile_row0, num_tiles, logits, ldz, ids, wts, top, over_all, wscale);
+                     tile_expert, tile_row0, num_tiles, logits, ldz, ids, wts, top, over_all, wscale, corr, outputs);
   SA_LAUNCH_CHECK();
   dim3 block(256);
   if (mfma) {
@@ -537,11 +596,12 @@ extern "C" int sa_moe_experts(const void* h, int act_dtype, int* ids, const void
 // Only the grouping (and, with logits, the routing): the lists for products that another library runs over tiles of
 // `tile_rows` grouped rows.  ints: as for sa_moe_experts, with max_tiles = sa_moe_max_tiles(T top, E).
 extern "C" int sa_moe_group(int* ids, int* ints, int T, int top, int E, int tile_rows, const float* logits, int ldz,
-                            float* wts, int over_all, float wscale, hipStream_t stream) {
+                            float* wts, int over_all, float wscale, const float* corr, int outputs, hipStream_t stream) {
   if (T <= 0) return 0;
   const long long n = (long long)T * top;
   if (E <= 0 || top <= 0 || tile_rows < 16 || n > 0x3fffffffLL) return SA_ERR_ARG;
-  if (logits && (T > MOE_ROUTE_INSIDE || !wts || ldz < E || top > E)) return SA_ERR_ARG;
+  if (logits && (T > MOE_ROUTE_INSIDE || !wts || outputs < E || ldz < outputs || top > outputs || (corr && over_all != 1)))
+    return SA_ERR_ARG;
   const int max_tiles = sa_moe_max_tiles((int)n, E);
   int* offsets = ints;
   int* cursor = offsets + E + 1;
@@ -550,22 +610,23 @@ extern "C" int sa_moe_group(int* ids, int* ints, int T, int top, int E, int tile
   int* tile_row0 = tile_expert + max_tiles;
   int* num_tiles = tile_row0 + max_tiles;
   hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, stream, ids, (int)n, E, tile_rows, offsets, cursor, perm,
-                     tile_expert, tile_row0, num_tiles, logits, ldz, ids, wts, top, over_all, wscale);
+                     tile_expert, tile_row0, num_tiles, logits, ldz, ids, wts, top, over_all, wscale, corr, outputs);
   SA_LAUNCH_CHECK();
   return 0;
 }
 
 extern "C" int sa_moe_combine(const float* yk, const float* wts, const void* shared, int shared_dtype, int parts,
-                              const float* sg, int ldz, float* y, int T, int top, int d, hipStream_t stream) {
+                              const float* sg, int ldz, float* y, int T, int top, int d, const int* ids, int E,
+                              const void* own, int own_dtype, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (top <= 0 || d <= 0 || parts < 1) return SA_ERR_ARG;
+  if (top <= 0 || d <= 0 || parts < 1 || (ids && (!own || (own_dtype != SA_F32 && own_dtype != SA_BF16)))) return SA_ERR_ARG;
   const size_t part_stride = (size_t)T * d;
   // a step of few rows: a value a thread, so that a row's loads are not a chain in one workgroup
   const int threads = d >= 256 ? 256 : 64;
   dim3 grid(T, T <= 64 ? (unsigned)((d + threads - 1) / threads) : 1u), block(threads);
 #define GO(TS, TOPMAX, PMAX)                                                                                       \
   hipLaunchKernelGGL((moe_combine_kernel<TS, TOPMAX, PMAX>), grid, block, 0, stream, yk, wts, (const TS*)shared,     \
-                     parts, part_stride, sg, ldz, y, top, d)
+                     parts, part_stride, sg, ldz, y, top, d, ids, E, own, own_dtype == SA_BF16 ? 1 : 0)
   const bool bounded = top <= 8 && parts <= 8;
   if (!shared || shared_dtype == SA_F32) {
     if (bounded) GO(float, 8, 8);

@@ -98,7 +98,9 @@ class Model:
     def _check_cache_owners(self) -> None:
         writers: Dict[int, int] = {}
         for e in self.spec.run_order:
-            if e.writes_cache:
+            if e.reads_pages_of is not None and e.writes_cache:
+                raise ValueError("an entry of the run order that reads another cache layer's pages does not write them")
+            if e.writes_cache or e.reads_pages_of is not None:
                 if e.cache in writers:
                     raise ValueError(f"cache layer {e.cache} is written by two entries of the run order")
                 writers[e.cache] = e.layer
@@ -107,6 +109,14 @@ class Model:
             if c not in writers:
                 raise ValueError(f"cache layer {c} is read but never written")
         self._cache_writer_layer = [writers[c] for c in range(n)]
+        written = set()
+        for e in self.spec.run_order:
+            if e.reads_pages_of is not None and e.reads_pages_of not in written:
+                raise ValueError(f"cache layer {e.reads_pages_of} is read before anything has written it")
+            if e.writes_cache:
+                written.add(e.cache)
+            elif e.reads_pages_of is not None and self._cache_owner(e.layer).cache_request() is not None:
+                raise ValueError(f"layer {e.layer} keeps keys of its own and cannot read another layer's")
 
     def _cache_owner(self, layer: int) -> Optional[Part]:
         return self.layers[layer].cache_owner()
@@ -155,7 +165,7 @@ class Model:
         reqs = self.cache_requests()
         out = []
         for e in self.spec.run_order:
-            r = reqs[e.cache]
+            r = reqs[e.cache if e.reads_pages_of is None else e.reads_pages_of]
             if r is not None:
                 out.append((sum(t.elements_per_token() for t in r.tensors), r.retention))
         return out
@@ -211,7 +221,10 @@ class Model:
                 ctx.next_input_norm = None          # (the stream changes between the two layers)
             if e.pass_vector is not None:
                 pending = self.pass_vectors.forward(x, pending, e.pass_vector, x0 if e.adds_embedding else None)
-            pending = self.layers[e.layer].forward(x, pending, ctx, caches[e.cache], e.writes_cache)
+            cache = caches[e.cache]
+            if e.reads_pages_of is not None:
+                cache = caches[e.reads_pages_of].with_state_of(cache)
+            pending = self.layers[e.layer].forward(x, pending, ctx, cache, e.writes_cache)
         if ctx.num_logit_rows == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=x.device)
         h = self.final_norm.forward(x, pending, rows=ctx.logit_rows)

@@ -94,7 +94,7 @@ def _i32(t: torch.Tensor, n: int, name: str) -> None:
 def embed(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor,
           src_row: Optional[torch.Tensor] = None, prev: Optional[torch.Tensor] = None,
           scale: float = 1.0) -> torch.Tensor:
-    """out[t] = table[tokens[t]] * scale as fp32 (the product is taken in fp32).  Where src_row[t] >= 0 the id is prev[src_row[t]] instead:
+    """out[t] = table[tokens[t]] * scale as fp32 (the product is taken in fp32); with out [T, S, d] S copies of it.  Where src_row[t] >= 0 the id is prev[src_row[t]] instead:
     a token sampled on the device by an earlier step.  Host-given ids have been checked against
     the table by the batch builder; the kernel clamps as a last resort."""
     _dev(table, tokens, out, src_row, prev)
@@ -102,13 +102,15 @@ def embed(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor,
     _check(table.dim() == 2, "embedding table must be [V, d]")
     V, d = table.shape
     _i32(tokens, T, "tokens")
-    _check(out.dtype == torch.float32 and out.shape == (T, d), "embed output must be fp32 [T, d]")
+    copies = out.shape[1] if out.dim() == 3 else 1
+    _check(out.dtype == torch.float32 and out.shape in ((T, d), (T, copies, d)) and copies > 0,
+           "embed output must be fp32 [T, d] or [T, copies, d]")
     if src_row is not None:
         _i32(src_row, T, "src_row")
         _check(prev is not None and prev.dtype == torch.int32, "prev must be int32")
     lib = load_library("elementwise")
     _ret(lib.sa_embed(_ptr(table), c_int(_code(table)), _ptr(tokens), _ptr(src_row), _ptr(prev), _ptr(out),
-                      c_int(T), c_int(d), c_int(V), c_float(scale), _stream()), "embed")
+                      c_int(T), c_int(d), c_int(V), c_float(scale), c_int(copies), _stream()), "embed")
     return out
 
 
@@ -1132,6 +1134,170 @@ def gated_average(rows: torch.Tensor, bias: torch.Tensor, state: torch.Tensor, c
 
 
 # ---------------------------------------------------------------------------------------------
+# a residual stream of several copies
+# ---------------------------------------------------------------------------------------------
+STREAM_MIX_MAX_STREAMS = 16
+STREAM_MIX_MAX_WIDTH = 16000
+
+
+@dataclass
+class ExpertRows:
+    """What a routed feed-forward leaves where its consumer adds the experts' rows up itself: yk fp32 [T top, d], weights
+    fp32 [T, top], ids int32 [T, top] (an id of `experts` or above: an identity expert, whose row is `own`'s [T, d])."""
+
+    yk: torch.Tensor
+    weights: torch.Tensor
+    ids: torch.Tensor
+    experts: int
+    own: torch.Tensor
+
+
+EXPERT_ROWS_MAX_TOP = 8          # (what `stream_mix` takes in its fast kernel)
+
+
+def stream_mix(x: torch.Tensor, y, bias: Optional[torch.Tensor], mix: Optional[torch.Tensor], to: Optional[torch.Tensor],
+               from_: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor,
+               rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Between two sublayers of a residual stream of S copies, x fp32 [T, S, d] in place:
+    x_t = sum_s mix[s, t] x_s + to[t] (y + bias), all copies at once from the old ones (y None: x stays), then
+    out = N(sum_t from_[t] x_t) * weight, N(u) = u / sqrt(mean(u^2) + eps).  y: [T, d] in out's dtype or fp32, fp32
+    [parts, T, d] partial sums added in order, or an `ExpertRows`.  mix [S, S], to [S], from_ [S], weight [d] and bias [d]
+    are fp32.  With `rows` only the listed rows are made (out[r] from source row rows[r]) and x is left as it was."""
+    _dev(x, bias, mix, to, from_, weight, out, rows)
+    _check(x.dtype == torch.float32 and x.dim() == 3, "the stream must be fp32 [T, S, d]")
+    T, S, d = x.shape
+    _check(0 < S <= STREAM_MIX_MAX_STREAMS and 0 < d <= STREAM_MIX_MAX_WIDTH,
+           f"up to {STREAM_MIX_MAX_STREAMS} copies of up to {STREAM_MIX_MAX_WIDTH} are taken")
+    R = T if rows is None else rows.numel()
+    if rows is not None:
+        _i32(rows, R, "rows")
+    _check(out.shape == (R, d), f"the output must be [{R}, {d}]")
+    _f32vec(from_, S, "the sublayer's input weights")
+    _f32vec(weight, d, "the norm's weight")
+    if bias is not None:
+        _f32vec(bias, d, "bias")
+    ids = wts = own = None
+    parts, ycode, row_stride, part_stride, experts, yt = 1, F32, d, 0, 0, None
+    if y is not None:
+        _check(mix is not None and to is not None, "an update needs its matrix and its output weights")
+        _f32vec(mix, S * S, "the streams' matrix")
+        _f32vec(to, S, "the output weights")
+        if isinstance(y, ExpertRows):
+            yt, wts, ids, own, experts = y.yk, y.weights, y.ids, y.own, y.experts
+            parts = wts.shape[1]
+            _dev(yt, wts, ids, own, x)
+            _check(yt.dtype == torch.float32 and yt.shape == (T * parts, d) and wts.dtype == torch.float32
+                   and wts.shape == (T, parts) and ids.dtype == torch.int32 and ids.shape == (T, parts)
+                   and own.shape == (T, d) and own.dtype == out.dtype,
+                   "expert rows: yk fp32 [T top, d], weights and ids [T, top], own rows in out's dtype")
+            row_stride, part_stride = parts * d, d
+        else:
+            yt = y
+            _dev(yt, x)
+            parts = _parts_of(y, T, d, "y")
+            _check(y.dtype in (out.dtype, torch.float32), "y must have out's dtype or be fp32")
+            part_stride = T * d
+            ycode = _code(y)
+    LL = ctypes.c_longlong
+    lib = load_library("stream_mix")
+    _ret(lib.sa_stream_mix(_ptr(x), c_int(S), _ptr(yt), c_int(ycode), LL(row_stride), LL(part_stride), c_int(parts),
+                           _ptr(wts), _ptr(ids), c_int(experts), _ptr(own), _ptr(bias if y is not None else None), _ptr(mix),
+                           _ptr(to), _ptr(from_), _ptr(weight), _ptr(out), c_int(_code(out)), _ptr(rows), c_float(eps), c_int(R),
+                           c_int(d), _stream()), "stream_mix")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------
+# attention behind a short convolution, and heads of several maps
+# ---------------------------------------------------------------------------------------------
+CONV_ATTENTION_MAX_TAPS = 16
+DIFFERENTIAL_MAX_VDIM = 640
+
+
+def conv_rope_kv_write(z: torch.Tensor, bias: Optional[torch.Tensor], conv_w: torch.Tensor, state: Optional[torch.Tensor],
+                       conv_offset: int, ctx, q_out: torch.Tensor, slots: Optional[torch.Tensor],
+                       k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], inv_freq: Optional[torch.Tensor],
+                       rot_dim: int, adjacent_pairs: bool, num_heads: int, num_kv_heads: int, maps: int, dim: int,
+                       vdim: int) -> torch.Tensor:
+    """From rows z [T, >= C], C channels [q: Hq M D | k: Hk M D | v: Hk Dv]: u = z + bias (fp32 [C] or None), then per channel
+    sum_j conv_w[c, j] u_(t - taps + 1 + j) over the segment's tokens, its request's earlier ones and zeros before position
+    0 (conv_w fp32 [C, taps]); in every map of every query and key head the first `rot_dim` dims rotated by
+    position * inv_freq[i] (pairs (2i, 2i + 1) with `adjacent_pairs`, else (i, i + rot_dim / 2)).  q_out [T, Hq M Dp]: every
+    (head, map) a row of Dp with its D dims in the map's places m D .. and zeros elsewhere; keys to k_pages [P, Hk, page, Dp],
+    a group's maps side by side and zeros behind; values to v_pages [P, Hk, Dp, page].  `slots` None: queries only (C = Hq M D).
+    `state` fp32 rows by ctx.state_slots: from `conv_offset` on the last taps - 1 rows of z, oldest first; updated here."""
+    T, B = ctx.num_tokens, ctx.num_segments
+    H, G, M, D, Dv = num_heads, num_kv_heads, maps, dim, vdim
+    _dev(bias, conv_w, q_out, slots, k_pages, v_pages, inv_freq, ctx.positions, ctx.seg_of_token, ctx.cu_q, ctx.state_slots)
+    write = slots is not None
+    C = H * M * D + (G * (M * D + Dv) if write else 0)
+    _rows(z, T, C, "z")
+    _check(conv_w.dtype == torch.float32 and conv_w.dim() == 2 and conv_w.shape[0] == C
+           and 1 <= conv_w.shape[1] <= CONV_ATTENTION_MAX_TAPS,
+           f"conv_w must be fp32 [{C}, taps] with up to {CONV_ATTENTION_MAX_TAPS} taps")
+    taps = conv_w.shape[1]
+    if bias is not None:
+        _f32vec(bias, C, "bias")
+    _check(q_out.dim() == 2 and q_out.shape[0] == T and q_out.shape[1] % (H * M) == 0 and q_out.dtype == z.dtype,
+           "q_out must be [T, Hq M Dp] in z's dtype")
+    Dp = q_out.shape[1] // (H * M)
+    _check(Dp >= M * D and Dp >= Dv, f"the padded head size {Dp} is below {M} x {D} or vdim {Dv}")
+    _check(rot_dim >= 0 and rot_dim % 2 == 0 and rot_dim <= D, "rot_dim must be even and within dim")
+    if rot_dim:
+        _check(inv_freq is not None, "a rotation needs its frequencies")
+        _f32vec(inv_freq, rot_dim // 2, "inv_freq")
+    ss = 0
+    if taps > 1:
+        _check(state is not None and state.is_cuda and state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+               and 0 <= conv_offset and conv_offset + (taps - 1) * C <= state.shape[1], "state rows are too short for the convolution")
+        ss = state.stride(0)
+    for name, n in (("positions", T), ("seg_of_token", T), ("cu_q", B + 1), ("state_slots", B)):
+        _i32(getattr(ctx, name), n, name)
+    page_size = 1
+    if write:
+        _i32(slots, T, "slots")
+        P, _, page_size, _ = k_pages.shape
+        _check(k_pages.shape == (P, G, page_size, Dp) and v_pages.shape == (P, G, Dp, page_size),
+               f"the cache must be k [P, {G}, page, {Dp}] and v [P, {G}, {Dp}, page]")
+        _check(k_pages.dtype == z.dtype and v_pages.dtype == z.dtype, "cache dtype must match activations")
+    lib = load_library("conv_attention")
+    LL = ctypes.c_longlong
+    single = int(getattr(ctx, "max_q_len", 0) or T) == 1
+    updated = c_int(0)
+    _ret(lib.sa_conv_rope_kv_write(
+        _ptr(z), LL(z.stride(0)), c_int(_code(z)), _ptr(bias), _ptr(conv_w), c_int(taps), _ptr(state if taps > 1 else None), LL(ss),
+        LL(conv_offset), _ptr(ctx.positions), _ptr(ctx.seg_of_token), _ptr(ctx.cu_q), _ptr(ctx.state_slots), _ptr(q_out),
+        _ptr(slots), _ptr(k_pages if write else None), _ptr(v_pages if write else None), _ptr(inv_freq if rot_dim else None),
+        c_int(rot_dim), c_int(1 if adjacent_pairs else 0), c_int(T), c_int(H), c_int(G), c_int(M), c_int(D), c_int(Dv), c_int(Dp),
+        c_int(page_size), c_int(1 if single else 0), ctypes.byref(updated), _stream()), "conv_rope_kv_write")
+    if not updated.value:
+        conv_state_update(z, 0, C, state, conv_offset, ctx, taps)
+    return q_out
+
+
+def differential_heads(a: torch.Tensor, gate_rows: Optional[torch.Tensor], gate_col: int, out: torch.Tensor, lam: float,
+                       scale: float, eps: float, num_heads: int, vdim: int) -> torch.Tensor:
+    """a [T, 2 H Dp], head h's two maps' outputs at 2 h and 2 h + 1 (Dv values and padding each): per head
+    o = a_1 - lam a_2, out[t, h, :] = o / sqrt(mean(o^2) + eps) * scale * sigmoid(gate_rows[t, gate_col + h Dv + i]) (fp32
+    arithmetic; gate_rows None: without the gate); out [T, H Dv]."""
+    _dev(a, out)
+    T, H, Dv = a.shape[0], num_heads, vdim
+    _check(a.dim() == 2 and a.shape[1] % (2 * H) == 0 and a.shape[1] // (2 * H) >= Dv, "a must be [T, 2 H Dp]")
+    _check(out.shape == (T, H * Dv) and out.dtype == a.dtype, "out must be [T, H Dv] in a's dtype")
+    _check(0 < Dv <= DIFFERENTIAL_MAX_VDIM, f"values of up to {DIFFERENTIAL_MAX_VDIM} are taken")
+    gs = 0
+    if gate_rows is not None:
+        _rows(gate_rows, T, gate_col + H * Dv, "gate rows")
+        _check(gate_rows.dtype == a.dtype, "the gate's logits must have a's dtype")
+        gs = gate_rows.stride(0)
+    lib = load_library("conv_attention")
+    _ret(lib.sa_differential_heads(_ptr(a), _ptr(gate_rows), ctypes.c_longlong(gs), c_int(gate_col), _ptr(out), c_int(_code(a)),
+                                   c_float(lam), c_float(scale), c_float(eps), c_int(T), c_int(H), c_int(Dv),
+                                   c_int(a.shape[1] // (2 * H)), _stream()), "differential_heads")
+    return out
+
+
+# ---------------------------------------------------------------------------------------------
 # routed experts
 # ---------------------------------------------------------------------------------------------
 
@@ -1148,20 +1314,28 @@ def _router_mode(over_all) -> int:
 
 
 def moe_route(logits: torch.Tensor, experts: int, top: int, ids: torch.Tensor, weights: torch.Tensor,
-              over_all=False, scale: float = 1.0) -> None:
-    """Per row of logits fp32 [T, >= experts]: the `top` experts with the largest logits (ids int32
+              over_all=False, scale: float = 1.0, correction: Optional[torch.Tensor] = None) -> None:
+    """Per row of logits fp32 [T, >= experts] (`experts`: all of the router's outputs): the `top` experts with the largest logits (ids int32
     [T, top]) and their weights fp32 [T, top]: the softmax over those logits alone ("chosen"), or (`over_all` True
     or "all") their shares of the softmax over all experts divided by the sum of the chosen shares + 1e-20, or
-    ("sigmoid") the sigmoid of each chosen logit, not normalised; times `scale`."""
-    _dev(logits, ids, weights)
+    ("sigmoid") the sigmoid of each chosen logit, not normalised; times `scale`.  `correction` (fp32 [experts], with "all"
+    only): those with the largest share + correction are chosen; the weights stay without it."""
+    _dev(logits, ids, weights, correction)
     T = logits.shape[0]
+    _check_correction(correction, experts, over_all)
     _check(logits.dtype == torch.float32 and logits.dim() == 2 and logits.shape[1] >= experts, "router logits must be fp32 [T, >= E]")
     _check(0 < top <= experts, "top must be within the number of experts")
     _check(ids.dtype == torch.int32 and ids.shape == (T, top) and weights.dtype == torch.float32 and weights.shape == (T, top),
            "ids int32 [T, top], weights fp32 [T, top]")
     lib = load_library("moe")
     _ret(lib.sa_moe_route(_ptr(logits), c_int(logits.shape[1]), _ptr(ids), _ptr(weights), c_int(T), c_int(experts),
-                          c_int(top), c_int(_router_mode(over_all)), c_float(scale), _stream()), "moe_route")
+                          c_int(top), c_int(_router_mode(over_all)), c_float(scale), _ptr(correction), _stream()), "moe_route")
+
+
+def _check_correction(correction: Optional[torch.Tensor], outputs: int, over_all) -> None:
+    if correction is not None:
+        _f32vec(correction, outputs, "the router's correction")
+        _check(_router_mode(over_all) == ROUTER_MODES["all"], "a correction goes with weights that are shares of the softmax over all")
 
 
 MOE_ROUTE_INSIDE = 16      # up to this many tokens the experts' call does the routing itself (one kernel less)
@@ -1179,14 +1353,17 @@ def moe_wide_available(h: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor
 def moe_experts(h: torch.Tensor, ids: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor,
                 yk: torch.Tensor, logits: Optional[torch.Tensor] = None,
                 weights: Optional[torch.Tensor] = None, over_all=False, scale: float = 1.0,
-                gate: str = "silu", limit: float = 0.0, weight_inputs: bool = False) -> torch.Tensor:
+                gate: str = "silu", limit: float = 0.0, weight_inputs: bool = False,
+                correction: Optional[torch.Tensor] = None, outputs: Optional[int] = None) -> torch.Tensor:
     """yk[t * top + k] = expert ids[t, k] applied to h[t]: down(gate(gate h, up h)), fp32 [T top, d], with
     one of GATES (silu(g) u unless said otherwise).
     w_gate, w_up [E, F, d], w_down [E, d, F] in h's dtype.  With `logits` (fp32 [T, >= E], at most
     MOE_ROUTE_INSIDE tokens) `ids` and `weights` are made here as `moe_route` makes them (`over_all`, `scale`).
     `weight_inputs`: expert ids[t, k] is applied to weights[t, k] * h[t] (the weight enters where the gate is applied,
-    gate and up being linear), for designs whose weights multiply the experts' inputs and not their outputs."""
-    _dev(h, ids, w_gate, w_up, w_down, yk, logits, weights)
+    gate and up being linear), for designs whose weights multiply the experts' inputs and not their outputs.
+    `outputs`: how many outputs the router has (None: E); ids of E and above are identity experts, whose rows of yk are
+    left alone (`moe_combine` and `stream_mix` take the token's own row for them).  `correction`: see `moe_route`."""
+    _dev(h, ids, w_gate, w_up, w_down, yk, logits, weights, correction)
     T, d = h.shape
     top = ids.shape[1]
     E, F, d2 = w_gate.shape
@@ -1196,6 +1373,9 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, w_gate: torch.Tensor, w_up: 
     _check(yk.dtype == torch.float32 and yk.shape == (T * top, d), "yk must be fp32 [T top, d]")
     _check(gate in GATES and (gate != "clamped_swish" or limit > 0.0), f"gate must be one of {sorted(GATES)}, "
            "the clamped one with a positive limit")
+    outputs = E if outputs is None else int(outputs)
+    _check(outputs >= E, "the router has an output for every expert")
+    _check_correction(correction, outputs, over_all)
     lib = load_library("moe")
     n = T * top
     tiles = int(lib.sa_moe_max_tiles(c_int(n), c_int(E)))
@@ -1209,7 +1389,7 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, w_gate: torch.Tensor, w_up: 
         wide = load_library("gemm_mfma")
         rows = int(wide.sa_moe_wide_tile_rows())
         _ret(lib.sa_moe_group(_ptr(ids), _ptr(ints), c_int(T), c_int(top), c_int(E), c_int(rows), c_void_p(0), c_int(0),
-                              c_void_p(0), c_int(0), c_float(1.0), _stream()), "moe_group")
+                              c_void_p(0), c_int(0), c_float(1.0), c_void_p(0), c_int(outputs), _stream()), "moe_group")
         base, o = ints.data_ptr(), 4
         offsets, perm = base, base + o * (2 * E + 1)
         tile_expert = perm + o * n
@@ -1222,23 +1402,26 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, w_gate: torch.Tensor, w_up: 
     ldz = 0
     if logits is not None:
         _check(T <= MOE_ROUTE_INSIDE and logits.dtype == torch.float32 and logits.dim() == 2 and logits.shape[0] == T
-               and logits.shape[1] >= E and 0 < top <= E, "moe_experts: logits fp32 [T, >= E] of at most "
+               and logits.shape[1] >= outputs and 0 < top <= outputs, "moe_experts: logits fp32 [T, >= outputs] of at most "
                f"{MOE_ROUTE_INSIDE} tokens")
         _check(weights is not None and weights.dtype == torch.float32 and weights.shape == (T, top), "weights fp32 [T, top]")
         ldz = logits.shape[1]
     _ret(lib.sa_moe_experts(_ptr(h), c_int(_code(h)), _ptr(ids), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(ints),
                             _ptr(act), _ptr(yk), c_int(T), c_int(top), c_int(E), c_int(d), c_int(F), _ptr(logits),
                             c_int(ldz), _ptr(weights), c_int(_router_mode(over_all)), c_float(scale), c_int(GATES[gate]),
-                            c_float(limit), _ptr(weights if weight_inputs else None), _stream()), "moe_experts")
+                            c_float(limit), _ptr(weights if weight_inputs else None), _ptr(correction), c_int(outputs), _stream()),
+         "moe_experts")
     return yk
 
 
 def moe_combine(yk: torch.Tensor, weights: Optional[torch.Tensor], shared: Optional[torch.Tensor],
-                logits: Optional[torch.Tensor], gate_col: int, y: torch.Tensor) -> torch.Tensor:
+                logits: Optional[torch.Tensor], gate_col: int, y: torch.Tensor, ids: Optional[torch.Tensor] = None,
+                experts: int = 0, own: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y[t] = sum_k weights[t, k] yk[t top + k] (+ sigmoid(logits[t, gate_col]) * shared[t]);
     shared [T, d] or fp32 [parts, T, d]; logits None: the shared rows are added as they are; weights None: the
-    experts' rows are added as they are."""
-    _dev(yk, weights, shared, logits, y)
+    experts' rows are added as they are.  `ids` (int32 [T, top]): where ids[t, k] >= `experts`, row t of `own` [T, d] takes
+    the place of yk[t top + k] (an identity expert)."""
+    _dev(yk, weights, shared, logits, y, ids, own)
     T, d = y.shape
     _check(T > 0 and yk.dim() == 2 and yk.shape[0] % T == 0, "moe_combine: yk must be [T top, d]")
     top = yk.shape[0] // T
@@ -1258,9 +1441,13 @@ def moe_combine(yk: torch.Tensor, weights: Optional[torch.Tensor], shared: Optio
         _check(logits.dtype == torch.float32 and logits.dim() == 2 and logits.shape[0] == T
                and 0 <= gate_col < logits.shape[1], "gate logits must be a column of fp32 [T, n]")
         gate, ldz = c_void_p(logits.data_ptr() + 4 * gate_col), logits.shape[1]
+    if ids is not None:
+        _check(ids.dtype == torch.int32 and ids.shape == (T, top), "ids must be int32 [T, top]")
+        _check(own is not None and own.shape == (T, d), "identity experts need the tokens' own rows [T, d]")
     lib = load_library("moe")
     _ret(lib.sa_moe_combine(_ptr(yk), _ptr(weights), _ptr(shared), c_int(scode), c_int(parts), gate,
-                            c_int(ldz), _ptr(y), c_int(T), c_int(top), c_int(d), _stream()), "moe_combine")
+                            c_int(ldz), _ptr(y), c_int(T), c_int(top), c_int(d), _ptr(ids), c_int(experts), _ptr(own),
+                            c_int(_code(own) if own is not None else F32), _stream()), "moe_combine")
     return y
 
 

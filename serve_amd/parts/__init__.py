@@ -4,3 +4,4 @@ from .base import (CacheTensor, LayerCache, ParamRequest, Part, PositionPart, Ro
 from . import standard  # noqa: F401
 from . import postnorm, recurrent, latent, feedforward, normed_attention  # noqa: F401
 from . import gated_attention, linear_recurrent, parallel, token_input, rotary_attention, gated_average  # noqa: F401
+from . import hyper_streams, differential_attention  # noqa: F401

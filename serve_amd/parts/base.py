@@ -19,8 +19,10 @@ Roles and what each must offer:
                 for per-request state of fixed size (`state_request`).  A mixer whose output has a
                 bias leaves it in `output_bias` (fp32 [d]) when it loads and says so before with
                 `has_output_bias`: the arrangement adds it to the stream (those that do: `adds_output_bias`).
-* feed_forward  `forward(h, ctx) -> delta [T, d]`.
-* embedding     `forward(ctx) -> x` fp32 [T, d] from the step's token ids (and whatever else of
+* feed_forward  `forward(h, ctx) -> delta [T, d]`.  One of routed experts may offer `leaves_rows` and is then asked with
+                `rows_ok=True` by consumers that add the experts' rows up themselves (`ops.ExpertRows`).
+* stream_weights  the weights of one sublayer on a residual stream of several copies (`hyper_streams`).
+* embedding     `forward(ctx) -> x` fp32 [T, d] (or [T, S, d]: a stream of S copies, for arrangements that know it) from the step's token ids (and whatever else of
                 the step it needs: positions for a learned position table).  An embedding that looks
                 back at a request's earlier tokens offers `state_request()` and is then called as
                 `forward(ctx, cache, keep=False)`: `cache.state` holds its row per request, and with
@@ -145,6 +147,10 @@ class LayerCache:
     def __post_init__(self):
         if self.pages is None:
             self.pages = {}
+
+    def with_state_of(self, other: "LayerCache") -> "LayerCache":
+        """These pages beside another cache layer's per-request state."""
+        return LayerCache(self.group, self.pages, self.page_size, other.state)
 
     @property
     def k_pages(self) -> Optional[torch.Tensor]:

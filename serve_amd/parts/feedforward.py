@@ -60,16 +60,24 @@ class RoutedExperts(Part):
     limit, if it differs).  `router_softmax="all"`: the weights are the chosen experts' shares of the softmax
     over all experts, divided by their sum (+ 1e-20); `"sigmoid"`: the weights are the sigmoids of the chosen
     logits as they are; `router_scale` multiplies the weights.  `weight_inputs`: a weight multiplies its expert's
-    input and not its output (the experts' outputs are then added as they are)."""
+    input and not its output (the experts' outputs are then added as they are).
+
+    `identity`: behind the experts the router has so many more outputs, whose expert is the token itself (its output is
+    the input, times the weight; they have no tensors).  `correction` (with `router_softmax="all"`): a stored number per
+    output is added to its share of the softmax where the experts are chosen, and not where they are weighted."""
 
     graph_safe = True
 
     def __init__(self, hidden_size: int, experts: int, top: int, expert_size: int,
                  shared_size: Optional[int] = None, shared_gate: bool = True, activation: str = "silu",
                  limit: float = 0.0, shared_limit: Optional[float] = None, router_softmax: str = "chosen",
-                 router_scale: float = 1.0, weight_inputs: bool = False):
-        if not 0 < top <= experts:
+                 router_scale: float = 1.0, weight_inputs: bool = False, identity: int = 0, correction: bool = False):
+        if identity < 0 or experts <= 0 or not 0 < top <= experts + identity:
             raise ValueError("top must be within the number of experts")
+        if correction and router_softmax != "all":
+            raise ValueError("a correction goes with weights that are shares of the softmax over all experts")
+        if identity and weight_inputs:
+            raise ValueError("an identity expert's weight multiplies its output")
         if router_softmax not in ops.ROUTER_MODES:
             raise ValueError(f"router_softmax must be one of {sorted(ops.ROUTER_MODES)}")
         if activation not in ops.GATES:
@@ -80,6 +88,10 @@ class RoutedExperts(Part):
         self.activation, self.limit = activation, float(limit)
         self.over_all, self.router_scale = router_softmax, float(router_scale)      # (the router's mode, by name)
         self.weight_inputs = bool(weight_inputs)
+        self.identity, self.correction = int(identity), bool(correction)
+        self.outputs = self.experts + self.identity           # the router's
+        # (a consumer may ask for the experts' rows as they are: nothing else is added to them here)
+        self.leaves_rows = not self.shared_size and not self.weight_inputs and self.top <= ops.EXPERT_ROWS_MAX_TOP
         self.shared = None
         if self.shared_size:
             self.shared = SwiGLU(self.hidden_size, self.shared_size, activation,
@@ -87,7 +99,9 @@ class RoutedExperts(Part):
 
     def param_requests(self) -> List[ParamRequest]:
         d, F = self.hidden_size, self.expert_size
-        out = [ParamRequest("router", (self.experts, d), init="normal:0.25")]
+        out = [ParamRequest("router", (self.outputs, d), init="normal:0.25")]
+        if self.correction:
+            out.append(ParamRequest("correction", (self.outputs,), init="normal:0.02"))
         for e in range(self.experts):
             out += [ParamRequest(f"e{e}.gate", (F, d), init="normal:0.08"), ParamRequest(f"e{e}.up", (F, d), init="normal:0.08"),
                     ParamRequest(f"e{e}.down", (d, F), init="normal:0.08")]
@@ -104,8 +118,10 @@ class RoutedExperts(Part):
         and as weights no more experts than the step's tokens can choose."""
         d, F = self.hidden_size, self.expert_size
         used = min(self.experts, tokens * self.top)
-        elements = self.experts * d + used * 3 * F * d
-        flops = 2.0 * tokens * self.experts * d + 2.0 * tokens * self.top * 3 * F * d
+        elements = self.outputs * d + used * 3 * F * d
+        flops = 2.0 * tokens * self.outputs * d
+        # (identity experts cost nothing; of a token's choices as many are theirs as of the outputs, on the average)
+        flops += 2.0 * tokens * self.top * (self.experts / self.outputs) * 3 * F * d
         if self.shared_size:
             elements += 3 * self.shared_size * d + (d if self.shared_gate else 0)
             flops += 2.0 * tokens * (3 * self.shared_size * d + (d if self.shared_gate else 0))
@@ -116,6 +132,7 @@ class RoutedExperts(Part):
         E = self.experts
         router = tensors["router"]
         rows = [router] + ([tensors["shared.sg"].to(router.dtype)] if self.shared_gate else [])
+        self.choice = tensors["correction"].float().contiguous() if self.correction else None
         self.w_router = torch.cat(rows, dim=0).contiguous()              # the shared expert's gate rides along
         dt = rt.dtype
         # (gates and ups in one tensor [2, E, F, d]: the kernel for many rows finds an expert's ups E F rows behind its gates)
@@ -127,7 +144,8 @@ class RoutedExperts(Part):
                               "down_proj.weight": tensors["shared.down"]}, rt)
         _prepare_products(rt, self.w_router)
 
-    def forward(self, h: torch.Tensor, ctx) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, ctx, rows_ok: bool = False):
+        """[T, d]; with `rows_ok`, where `leaves_rows` says so, an `ops.ExpertRows` that the caller adds up."""
         T, d = h.shape
         dev = h.device
         logits = linear(h, self.w_router, out_dtype=torch.float32)
@@ -136,15 +154,19 @@ class RoutedExperts(Part):
         yk = torch.empty((T * self.top, d), dtype=torch.float32, device=dev)
         if T <= ops.MOE_ROUTE_INSIDE:
             ops.moe_experts(h, ids, self.w_gate, self.w_up, self.w_down, yk, logits, weights, self.over_all,
-                            self.router_scale, self.activation, self.limit, self.weight_inputs)    # routes, too
+                            self.router_scale, self.activation, self.limit, self.weight_inputs, self.choice,
+                            self.outputs)    # routes, too
         else:
-            ops.moe_route(logits, self.experts, self.top, ids, weights, self.over_all, self.router_scale)
+            ops.moe_route(logits, self.outputs, self.top, ids, weights, self.over_all, self.router_scale, self.choice)
             ops.moe_experts(h, ids, self.w_gate, self.w_up, self.w_down, yk, weights=weights, gate=self.activation,
-                            limit=self.limit, weight_inputs=self.weight_inputs)
+                            limit=self.limit, weight_inputs=self.weight_inputs, outputs=self.outputs)
+        if rows_ok and self.leaves_rows:
+            return ops.ExpertRows(yk, weights, ids, self.experts, h)
         shared = self.shared.forward(h, ctx) if self.shared is not None else None
         y = torch.empty((T, d), dtype=torch.float32, device=dev)
         return ops.moe_combine(yk, None if self.weight_inputs else weights, shared,
-                               logits if self.shared_gate else None, self.experts, y)
+                               logits if self.shared_gate else None, self.outputs, y,
+                               ids if self.identity else None, self.experts, h if self.identity else None)
 
 
 register_part("feed_forward", "dense", DenseFeedForward)

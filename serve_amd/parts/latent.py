@@ -13,7 +13,8 @@ window and scale.
 
 Options: `q_rank`: the queries go through a latent of their own, q = W_uq (N(W_dq h) w_dq) (tensors `dq`, `dq.norm`,
 `uq` in place of `q`); `out_gate`: the concatenated heads are multiplied element by element with sigmoid(W_g h) before
-W_o.  The rotation of the shared key part may pair (i, i + rot_dim / 2) or (2i, 2i + 1): queries and keys are only ever
+W_o, or (`out_gate="head"`) head h's output with the one number sigmoid(W_g h)_h, whose row of W_g rides behind the
+queries in their product.  The rotation of the shared key part may pair (i, i + rot_dim / 2) or (2i, 2i + 1): queries and keys are only ever
 multiplied with each other, so the second kind is the first after the rows of the projections that make the rotated
 parts have been put into the order (even places, odd places), which is done when the part loads.  A rotation with a
 magnitude (sine and cosine times a constant) is carried out by the kernels.
@@ -39,14 +40,18 @@ class LatentAttention(Part):
 
     def __init__(self, hidden_size: int, heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, scale: float,
                  eps: float, position: PartSpec, window: Optional[int] = None, retain: Optional[int] = None,
-                 own_kv: bool = True, q_rank: Optional[int] = None, out_gate: bool = False):
+                 own_kv: bool = True, q_rank: Optional[int] = None, out_gate=False):
         """`window`: a query at position i sees keys j with 0 <= i - j < window (None: all).  `retain`:
         how many keys the cache keeps (None: all): at least the window, and more if another layer
         with a longer window reads this layer's cache."""
         self.hidden_size, self.heads, self.dim, self.rot_dim = int(hidden_size), int(heads), int(dim), int(rot_dim)
         self.vdim, self.kv_rank, self.scale, self.eps = int(vdim), int(kv_rank), float(scale), float(eps)
         self.window, self.retain, self.own_kv = window, retain, bool(own_kv)
-        self.q_rank, self.out_gate = None if not q_rank else int(q_rank), bool(out_gate)
+        self.q_rank = None if not q_rank else int(q_rank)
+        if out_gate not in (False, True, "head"):
+            raise ValueError(f"out_gate is True (element by element), 'head' or False, got {out_gate!r}")
+        self.head_gate = out_gate == "head"
+        self.out_gate = bool(out_gate) and not self.head_gate
         if self.rot_dim % 2:
             raise ValueError("rot_dim must be even")
         if window is not None and retain is not None and retain < window:
@@ -69,6 +74,8 @@ class LatentAttention(Part):
             out = [ParamRequest("q", (H * (self.dim + self.rot_dim), d), init="normal:0.08")]
         if self.out_gate:
             out.append(ParamRequest("g", (H * self.vdim, d), init="normal:0.08"))
+        if self.head_gate:
+            out.append(ParamRequest("g", (H, d), init="normal:0.08"))
         if self.own_kv:
             out += [ParamRequest("dkv", (R + self.rot_dim, d), init="normal:0.07"),
                     ParamRequest("dkv.norm", (R,), init="ones_normal:0.15")]
@@ -114,6 +121,14 @@ class LatentAttention(Part):
             self.q_norm = tensors["dq.norm"].float().contiguous()
         self.w_g = tensors["g"] if self.out_gate else None
         dt = self.wq.dtype
+        self.gate_col = -1                       # where the heads' gate logits lie behind the queries (-1: elsewhere)
+        if self.head_gate and not self.q_rank and tensors["g"].dtype == dt:
+            n = self.wq.shape[0] + H
+            pad = torch.zeros((-n % 8, self.hidden_size), dtype=dt, device=self.wq.device)       # (rows of whole vectors)
+            self.gate_col = self.wq.shape[0]
+            self.wq = torch.cat([self.wq, tensors["g"], pad], dim=0).contiguous()
+        elif self.head_gate:
+            self.w_g = tensors["g"]
         # [H, dim, R]: the queries' way into the latent space; [H, R, vdim]: the latents' way out
         self.w_uk = tensors["uk"].to(dt).view(H, self.dim, R).contiguous()
         self.w_uv = tensors["uv"].to(dt).view(H, self.vdim, R).transpose(1, 2).contiguous()
@@ -157,6 +172,8 @@ class LatentAttention(Part):
         ops.head_linear(attn, H * D, D, self.w_uv, o, H * self.vdim, self.vdim, T)
         if self.out_gate:
             ops.sigmoid_mul(o, linear(h, self.w_g))
+        elif self.head_gate:
+            ops.head_gate(o, *((q, self.gate_col) if self.gate_col >= 0 else (linear(h, self.w_g), 0)), H)
         return linear(o, self.wo, partial_ok=True)
 
 

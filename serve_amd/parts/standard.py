@@ -313,13 +313,14 @@ class TokenEmbedding(Part):
 
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, side_width: int = 0):
+    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, side_width: int = 0,
+                 copies: int = 0):
         """`scale` multiplies every row as it enters the stream (in fp32; the table itself, which an
         output head may share, stays as stored).  `side_width` > 0: the part also holds a second table
         `side` [vocab, side_width], a second row per token that parts of the layers read (they name it as
-        `embedding.side`); nothing of it enters the stream here."""
+        `embedding.side`); nothing of it enters the stream here.  `copies` > 0: the stream is [T, copies, d], equal copies."""
         self.vocab_size, self.hidden_size, self.scale = int(vocab_size), int(hidden_size), float(scale)
-        self.side_width = int(side_width)
+        self.side_width, self.copies = int(side_width), int(copies)
 
     def param_requests(self) -> List[ParamRequest]:
         out = [ParamRequest("weight", (self.vocab_size, self.hidden_size))]
@@ -340,7 +341,8 @@ class TokenEmbedding(Part):
     def forward(self, ctx) -> torch.Tensor:
         """The rows of the step's tokens.  `ctx.src_row` / `ctx.prev_tokens` (when set): rows whose
         token was sampled on the device by an earlier step and never reached the host."""
-        x = self.rt.empty((ctx.token_ids.numel(), self.hidden_size), torch.float32)
+        T = ctx.token_ids.numel()
+        x = self.rt.empty((T, self.copies, self.hidden_size) if self.copies else (T, self.hidden_size), torch.float32)
         return ops.embed(self.weight, ctx.token_ids, x, ctx.src_row, ctx.prev_tokens, self.scale)
 
 

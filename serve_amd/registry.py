@@ -25,7 +25,7 @@ _ARCHITECTURES: Dict[str, Architecture] = {}
 _PARTS: Dict[Tuple[str, str], type] = {}
 
 PART_ROLES = ("mixer", "feed_forward", "norm", "position", "embedding", "lm_head", "arrangement", "token_input",
-              "stream_input")
+              "stream_input", "stream_weights")
 
 
 def register_architecture(name: str, config_from_dict, build_spec) -> None:
@@ -88,3 +88,4 @@ def _ensure_builtin() -> None:
         from .models import kotipel  # noqa: F401  (registers Kotipel)
         from .models import robuvik  # noqa: F401  (registers Robuvik)
         from .models import topapel  # noqa: F401  (registers Topapel)
+        from .models import befirax  # noqa: F401  (registers Befirax)
