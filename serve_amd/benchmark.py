@@ -179,10 +179,42 @@ SHAPES.update({
     "topapel-2k": _topapel_shape(2048, 32768, 8, 32, 8, 64, 1024, 2048, 16, 128, 8192),
     "topapel-4k": _topapel_shape(4096, 32768, 4, 32, 8, 128, 1024, 4096, 32, 128, 14336),
 })
+
+
+def _befirax_shape(width: int, vocab: int, layers: int, streams: int, heads: int, kv_heads: int, dim: int, vdim: int,
+                   lat_heads: int, window: int, ssm_heads: int, experts: int, identity: int, top: int, expert_ff: int):
+    """A Befirax shape at the sizes of a real model's layers: in turn a differential attention (`heads` on `kv_heads` heads of
+    two maps of `dim`, half of whose dims are rotated, values of `vdim`, four taps), a latent attention (`lat_heads` heads of
+    64 + 32 rotated dims over a latent of 96: a cache row as wide as the matrix-core attention's widest head; a window), a
+    state-space layer (inner width twice the model's: `ssm_heads` heads of 64, state 128, four taps) and a differential
+    attention on the keys and values of the first, each with routed experts some of which are the identity; `streams` copies
+    of the residual stream."""
+    from .config.befirax import (BefiraxConfig, BefiraxLayerConfig, DifferentialAttentionConfig, IdentityMoeConfig, PlainRotConfig,
+                                 WindowedLatentConfig)
+    from .config.kotipel import StateSpaceMixerConfig
+    rot = PlainRotConfig(500000.0, dim // 2)
+    moe = IdentityMoeConfig(experts, identity, top, expert_ff)
+    out = []
+    for i in range(layers):
+        mixer = (DifferentialAttentionConfig(heads, kv_heads, dim, vdim, dim ** -0.5, 0.5, 4, rot),
+                 WindowedLatentConfig(lat_heads, 64, 32, 64, 96, 96 ** -0.5, PlainRotConfig(1.0e6, 32), window),
+                 StateSpaceMixerConfig(ssm_heads, 64, 128, 1, 4, 1),
+                 DifferentialAttentionConfig(heads, kv_heads, dim, vdim, dim ** -0.5, 0.6, 4, rot, i - 3))[i % 4]
+        out.append(BefiraxLayerConfig(mixer, moe))
+    return BefiraxConfig(vocab=vocab, width=width, eps=1e-5, streams=streams, layers=tuple(out))
+
+
+# Befirax at the same two widths, depths and vocabularies; its attention has as many query, key and value columns as the
+# Llama shapes' (two maps of 64 and values of 128 where they have heads), its experts are Zozosun's and Timopel's
+SHAPES.update({
+    "befirax-tiny": _befirax_shape(64, 512, 4, 2, 2, 1, 16, 32, 2, 24, 2, 4, 2, 2, 32),
+    "befirax-2k": _befirax_shape(2048, 32768, 8, 4, 16, 4, 64, 128, 16, 1024, 64, 32, 8, 4, 1024),
+    "befirax-4k": _befirax_shape(4096, 32768, 4, 4, 32, 8, 64, 128, 32, 1024, 128, 64, 16, 6, 1536),
+})
 DESIGN_PAIRS = (("zozosun-2k", "llama-2k"), ("zozosun-4k", "llama-4k"), ("timopel-2k", "llama-2k"),
                 ("timopel-4k", "llama-4k"), ("kotipel-2k", "llama-2k"), ("kotipel-4k", "llama-4k"),
                 ("robuvik-2k", "llama-2k"), ("robuvik-4k", "llama-4k"), ("topapel-2k", "llama-2k"),
-                ("topapel-4k", "llama-4k"))
+                ("topapel-4k", "llama-4k"), ("befirax-2k", "llama-2k"), ("befirax-4k", "llama-4k"))
 
 
 def generate_requests(input_length: int, output_length: int, num_sequences: int, vocab_size: int,

@@ -18,6 +18,8 @@
 #include "common.h"
 
 #define CA_MAX_TAPS 16
+#define CA_RUN 4                  // consecutive tokens a thread of the prompt kernel takes (4 or 8; 8 was slower by 1 us of 11)
+#define CA_THREADS 64             // (with 256: slower by 1 to 2 us of 11)
 
 struct ConvRows {
   const float* bias;          // [C] or null
@@ -128,7 +130,7 @@ __global__ __launch_bounds__(256) void conv_rope_kv_write_kernel(
 // bf16, pairs (2i, 2i + 1), up to 4 taps, D, Dv, Dp and the row stride multiples of 8, aligned arrays: a thread takes eight
 // channels of TT consecutive tokens, so that a row of z is loaded once per TT tokens and thread (and taps - 1 rows in front
 // of them).  TT 1: steps of single tokens, which also leave their rows in the state (`update`: every segment is one token).
-// Threads whose eight places are padding write zeros.  Rows of z and the state's (copies of earlier rows of z) are kept as
+// Zeros of the padding are written by the threads that hold the row's data.  Rows of z and the state's (copies of earlier rows of z) are kept as
 // the bf16 bits they are.
 // ---------------------------------------------------------------------------------------------
 __device__ __forceinline__ void ca_unpack8(const uint4& v, float* f) {
@@ -139,12 +141,15 @@ __device__ __forceinline__ void ca_unpack8(const uint4& v, float* f) {
     f[2 * k + 1] = bf16_bits_to_float(w[k] >> 16);
   }
 }
+typedef __bf16 ca_bf16x2_t __attribute__((ext_vector_type(2)));
+typedef float ca_float2_t __attribute__((ext_vector_type(2)));
+// two floats to two bf16 (round to nearest even) in one v_cvt_pk_bf16_f32
+__device__ __forceinline__ uint32_t ca_pack2(float a, float b) {
+  const ca_float2_t f = {a, b};
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f, ca_bf16x2_t));
+}
 __device__ __forceinline__ uint4 ca_pack8(const float* f) {
-  uint32_t w[4];
-#pragma unroll
-  for (int k = 0; k < 4; ++k)
-    w[k] = (uint32_t)float_to_bf16_bits(f[2 * k]) | ((uint32_t)float_to_bf16_bits(f[2 * k + 1]) << 16);
-  return make_uint4(w[0], w[1], w[2], w[3]);
+  return make_uint4(ca_pack2(f[0], f[1]), ca_pack2(f[2], f[3]), ca_pack2(f[4], f[5]), ca_pack2(f[6], f[7]));
 }
 
 __device__ __forceinline__ void ca_load8(const float* __restrict__ p, float* f) {
@@ -154,48 +159,46 @@ __device__ __forceinline__ void ca_load8(const float* __restrict__ p, float* f) 
 }
 
 template <int TAPS, int TT>
-__global__ __launch_bounds__(256) void conv_rope_kv_write_vec_kernel(
+__global__ __launch_bounds__(CA_THREADS) void conv_rope_kv_write_vec_kernel(
     const bf16_t* __restrict__ z, long long zs, ConvRows in, bf16_t* __restrict__ q_out, const int* __restrict__ slot,
     bf16_t* __restrict__ k_pages, bf16_t* __restrict__ v_pages, const float* __restrict__ freq, int rot, int T, int H, int G,
     int M, int D, int Dv, int Dp, int page_size, int update) {
-  const int cph = Dp >> 3;
-  const int qv = H * M * cph, kv = slot ? G * cph : 0;
+  // data vectors of eight places: a (head, map) has D / 8, a group's keys M D / 8, its values Dv / 8
+  const int nq = D >> 3, nk = M * nq, nv = Dv >> 3, row = Dp >> 3;
+  const int qv = H * M * nq, kv = slot ? G * nk : 0, vv_ = slot ? G * nv : 0;
   const int item = blockIdx.x * blockDim.x + threadIdx.x;
-  if (item >= qv + 2 * kv) return;
+  if (item >= qv + kv + vv_) return;
   const int t0 = blockIdx.y * TT;
   const int nt = min(TT, T - t0);
   const bool is_q = item < qv, is_k = !is_q && item < qv + kv;
   const int rel = is_q ? item : (is_k ? item - qv : item - qv - kv);
-  const int u = rel / cph, i0 = (rel - u * cph) * 8;                  // (head, map) or group; first place
-  int c = -1, e0 = 0;                                                 // first channel (-1: padding), its dim in the map
-  if (is_q) {
-    const int first = (u % M) * D;
-    if (i0 >= first && i0 < first + D) { e0 = i0 - first; c = u * D + e0; }
-  } else if (is_k) {
-    if (i0 < M * D) { e0 = i0 % D; c = H * M * D + u * M * D + i0; }
-  } else if (i0 < Dv) {
-    c = (H + G) * M * D + u * Dv + i0;
-  }
+  const int per = is_q ? nq : (is_k ? nk : nv);
+  const int u = rel / per, mine = rel - u * per;                     // (head, map) or group; which of its vectors
+  const int first = is_q ? (u % M) * nq : 0;                         // the row's vector at which the data begin
+  const int i0 = (first + mine) * 8;
+  const int e0 = (is_k ? i0 % D : mine * 8);                         // the first dim inside its map
+  const int c = (is_q ? u * D : (is_k ? H * M * D + u * M * D : (H + G) * M * D + u * Dv)) + mine * 8;      // first channel
   const uint4 none = make_uint4(0u, 0u, 0u, 0u);
-  if (c < 0) {
+  // the rest of a row is zeros: its vectors are dealt to the threads that hold the row's data
+  if (row > per) {
     for (int n = 0; n < nt; ++n) {
       const int t = t0 + n;
-      if (is_q) {
-        *reinterpret_cast<uint4*>(q_out + ((size_t)t * H * M + u) * Dp + i0) = none;
-        continue;
-      }
-      const int s = slot[t];
+      const int s = is_q ? 0 : slot[t];
       if (s < 0) continue;
       const int page = s / page_size, off = s - page * page_size;
-      if (is_k) {
-        *reinterpret_cast<uint4*>(k_pages + (((size_t)page * G + u) * page_size + off) * Dp + i0) = none;
-      } else {
-        bf16_t* vp = v_pages + (((size_t)page * G + u) * Dp + i0) * page_size + off;
+      for (int j = mine; j < row - per; j += per) {
+        const int at = (j < first ? j : j + per) * 8;
+        if (is_q) {
+          *reinterpret_cast<uint4*>(q_out + ((size_t)t * H * M + u) * Dp + at) = none;
+        } else if (is_k) {
+          *reinterpret_cast<uint4*>(k_pages + (((size_t)page * G + u) * page_size + off) * Dp + at) = none;
+        } else {
+          bf16_t* vp = v_pages + (((size_t)page * G + u) * Dp + at) * page_size + off;
 #pragma unroll
-        for (int k = 0; k < 8; ++k) vp[(size_t)k * page_size].v = 0;
+          for (int k = 0; k < 8; ++k) vp[(size_t)k * page_size].v = 0;
+        }
       }
     }
-    return;
   }
   float w[8][TAPS], b[8];
 #pragma unroll
@@ -269,16 +272,16 @@ __global__ __launch_bounds__(256) void conv_rope_kv_write_vec_kernel(
       raw[TAPS - 1 + n] = *reinterpret_cast<const uint4*>(z + (size_t)(t0 + n) * zs + c);
       live[TAPS - 1 + n] = true;
     }
-    // values whose tokens lie side by side in one page leave as 16 bytes a channel
+    // values whose tokens lie side by side in one page leave as one vector a channel
     bool side_by_side = false;
     int s0 = -1;
-    if (TT == 8 && !is_q && !is_k) {
+    if (!is_q && !is_k) {
       s0 = slot[t0];
-      side_by_side = s0 >= 0 && (s0 & 7) == 0 && (page_size & 7) == 0;
+      side_by_side = s0 >= 0 && (s0 & (TT - 1)) == 0 && (page_size & (TT - 1)) == 0;
 #pragma unroll
       for (int n = 1; n < TT; ++n) side_by_side = side_by_side && slot[t0 + n] == s0 + n;
     }
-    uint32_t vv[8][4];
+    uint32_t vv[8][TT / 2 > 0 ? TT / 2 : 1];
 #pragma unroll
     for (int n = 0; n < TT; ++n) {
       float o[8];
@@ -296,8 +299,8 @@ __global__ __launch_bounds__(256) void conv_rope_kv_write_vec_kernel(
 #pragma unroll
         for (int k = 0; k < 8; ++k) {
           const uint32_t bits = float_to_bf16_bits(o[k]);
-          if (n & 1) vv[k][(n >> 1) & 3] |= bits << 16;
-          else vv[k][(n >> 1) & 3] = bits;
+          if (n & 1) vv[k][n >> 1] |= bits << 16;
+          else vv[k][n >> 1] = bits;
         }
       } else {
         store(t0 + n, pos0 + n, o);
@@ -307,8 +310,10 @@ __global__ __launch_bounds__(256) void conv_rope_kv_write_vec_kernel(
       const int page = s0 / page_size, off = s0 - page * page_size;
       bf16_t* vp = v_pages + (((size_t)page * G + u) * Dp + i0) * page_size + off;
 #pragma unroll
-      for (int k = 0; k < 8; ++k)
-        *reinterpret_cast<uint4*>(vp + (size_t)k * page_size) = make_uint4(vv[k][0], vv[k][1], vv[k][2], vv[k][3]);
+      for (int k = 0; k < 8; ++k) {
+        if constexpr (TT == 8) *reinterpret_cast<uint4*>(vp + (size_t)k * page_size) = make_uint4(vv[k][0], vv[k][1], vv[k][2], vv[k][3]);
+        else if constexpr (TT == 4) *reinterpret_cast<uint2*>(vp + (size_t)k * page_size) = make_uint2(vv[k][0], vv[k][1]);
+      }
     }
     return;
   }
@@ -374,11 +379,11 @@ extern "C" int sa_conv_rope_kv_write(const void* z, long long zs, int act_dtype,
   const ConvRows in = {bias, w, state, state_stride, conv_off, positions, seg_of_token, cu_q, state_slots, taps, C};
   const uintptr_t at = (uintptr_t)z | (uintptr_t)q_out | (slot ? (uintptr_t)k_pages | (uintptr_t)v_pages : 0);
   if (conv_vec_fits(act_dtype, zs, in, rot, adjacent, D, Dv, Dp, at)) {
-    const int items = (H * M + (slot ? 2 * G : 0)) * (Dp >> 3);
-    const int tt = single_tokens || T < 512 ? 1 : 8;
+    const int items = (H * M * D + (slot ? G * (M * D + Dv) : 0)) >> 3;
+    const int tt = single_tokens || T < 512 ? 1 : CA_RUN;
     const long long gy = ((long long)T + tt - 1) / tt;
     if (gy > 65535) return SA_ERR_ARG;
-    dim3 grid((items + 255) / 256, (unsigned)gy), block(256);
+    dim3 grid((items + CA_THREADS - 1) / CA_THREADS, (unsigned)gy), block(CA_THREADS);
 #define GO(TAPS_, TT_)                                                                                                     \
   hipLaunchKernelGGL((conv_rope_kv_write_vec_kernel<TAPS_, TT_>), grid, block, 0, stream, (const bf16_t*)z, zs, in,          \
                      (bf16_t*)q_out, slot, (bf16_t*)k_pages, (bf16_t*)v_pages, freq, rot, T, H, G, M, D, Dv, Dp, page_size, \
@@ -386,7 +391,7 @@ extern "C" int sa_conv_rope_kv_write(const void* z, long long zs, int act_dtype,
 #define GO_TT(TAPS_)           \
   do {                         \
     if (tt == 1) GO(TAPS_, 1); \
-    else GO(TAPS_, 8);         \
+    else GO(TAPS_, CA_RUN);    \
   } while (0)
     if (taps == 1) GO_TT(1);
     else if (taps == 2) GO_TT(2);

@@ -10,7 +10,8 @@
 //   head_linear       out[t, h, :] = in[t, h, :] W[h]  (W [H, K, N]): the queries into the latent
 //                     space, and the latent outputs out of it
 //                     (behind a head's outputs it can put the rotated part of the query and the row's padding,
-//                     so that the queries are one kernel)
+//                     so that the queries are one kernel; and it can multiply a head's outputs by sigmoid of one logit
+//                     a token and head, an output gate)
 //
 // Rotation: dimension i of the rotated part is paired with i + dr/2; (u, v) -> (u cos a - v sin a,
 // v cos a + u sin a), a = position * inv_freq[i], in fp32.
@@ -23,20 +24,20 @@ __device__ __forceinline__ void sincos_for(float a, float* sn, float* cs) {
 }
 
 // ---------------------------------------------------------------------------------------------
-// z [T, R + dr] -> k_pages [P, 1, page, Dp] rows [c | kr | 0], v_pages [P, 1, Dp, page] columns [c | 0].
+// z rows [T, >= R + dr], zs elements apart -> k_pages [P, 1, page, Dp] rows [c | kr | 0], v_pages [P, 1, Dp, page] columns [c | 0].
 // slot[t] = page * page_size + offset, < 0: nothing stored.  One workgroup a token.
 // ---------------------------------------------------------------------------------------------
 template <typename TA>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(
     const TA* __restrict__ z, const float* __restrict__ w, const int* __restrict__ positions,
     const float* __restrict__ inv_freq, const int* __restrict__ slot, TA* __restrict__ k_pages,
-    TA* __restrict__ v_pages, float eps, int R, int dr, int Dp, int page_size, float magnitude) {
+    TA* __restrict__ v_pages, float eps, int R, int dr, int Dp, int page_size, float magnitude, long long zs) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const int s = slot[t];
   if (s < 0) return;                       // (uniform over the workgroup)
   const int page = s / page_size, off = s - page * page_size;
-  const TA* zr = z + (size_t)t * (R + dr);
+  const TA* zr = z + (size_t)t * zs;
   float ss = 0.f;
   for (int i = threadIdx.x; i < R; i += blockDim.x) {
     const float v = to_float(zr[i]);
@@ -67,16 +68,17 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
 
 extern "C" int sa_latent_kv_write(const void* z, int act_dtype, const float* w, const int* positions,
                                   const float* inv_freq, const int* slot, void* k_pages, void* v_pages, float eps,
-                                  int T, int R, int dr, int Dp, int page_size, float magnitude, hipStream_t stream) {
+                                  int T, int R, int dr, int Dp, int page_size, float magnitude, long long zs,
+                                  hipStream_t stream) {
   if (T <= 0) return 0;
-  if (R <= 0 || dr < 0 || (dr & 1) || Dp < R + dr || page_size <= 0) return SA_ERR_ARG;
+  if (zs < R + dr || R <= 0 || dr < 0 || (dr & 1) || Dp < R + dr || page_size <= 0) return SA_ERR_ARG;
   dim3 grid(T), block(Dp > 128 ? 256 : 64);
   if (act_dtype == SA_F32)
     hipLaunchKernelGGL(latent_kv_write_kernel<float>, grid, block, 0, stream, (const float*)z, w, positions, inv_freq,
-                       slot, (float*)k_pages, (float*)v_pages, eps, R, dr, Dp, page_size, magnitude);
+                       slot, (float*)k_pages, (float*)v_pages, eps, R, dr, Dp, page_size, magnitude, zs);
   else if (act_dtype == SA_BF16)
     hipLaunchKernelGGL(latent_kv_write_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)z, w, positions,
-                       inv_freq, slot, (bf16_t*)k_pages, (bf16_t*)v_pages, eps, R, dr, Dp, page_size, magnitude);
+                       inv_freq, slot, (bf16_t*)k_pages, (bf16_t*)v_pages, eps, R, dr, Dp, page_size, magnitude, zs);
   else return SA_ERR_UNSUPPORTED;
   SA_LAUNCH_CHECK();
   return 0;
@@ -97,6 +99,16 @@ struct HeadTail {
   const float* inv_freq;     // [rot / 2]
   int rot, tail;
   float magnitude;           // multiplies sine and cosine
+};
+
+// An output gate: head h's outputs of token t times sigmoid(rows[t * stride + h]); rows null: none.
+template <typename TA>
+struct HeadGate {
+  const TA* rows;
+  long long stride;
+  __device__ __forceinline__ float at(int t, int h) const {
+    return rows ? 1.f / (1.f + expf(-to_float(rows[(size_t)t * stride + h]))) : 1.f;
+  }
 };
 
 template <typename TA>
@@ -120,7 +132,7 @@ __device__ __forceinline__ void write_tail(const HeadTail& ht, const TA* __restr
 template <typename TA>
 __global__ __launch_bounds__(256) void head_linear_kernel(const TA* __restrict__ in, int is, int ihs,
                                                           const TA* __restrict__ W, TA* __restrict__ out, int os,
-                                                          int ohs, int T, int K, int N, HeadTail ht) {
+                                                          int ohs, int T, int K, int N, HeadTail ht, HeadGate<TA> hg) {
   __shared__ float sin_[HL_TT][HL_KC];
   const int t0 = blockIdx.x * HL_TT;
   const int h = blockIdx.y;
@@ -148,7 +160,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const TA* __restrict__
   if (n < N) {
 #pragma unroll
     for (int tt = 0; tt < HL_TT; ++tt)
-      if (t0 + tt < T) out[(size_t)(t0 + tt) * os + (size_t)h * ohs + n] = from_float<TA>(acc[tt]);
+      if (t0 + tt < T) out[(size_t)(t0 + tt) * os + (size_t)h * ohs + n] = from_float<TA>(acc[tt] * hg.at(t0 + tt, h));
   }
   if (ht.positions && blockIdx.z == 0) {
     for (int tt = 0; tt < HL_TT && t0 + tt < T; ++tt)
@@ -165,7 +177,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const TA* __restrict__
 template <typename TA>
 __global__ __launch_bounds__(256) void head_linear_small_kernel(const TA* __restrict__ in, int is, int ihs,
                                                                 const TA* __restrict__ W, TA* __restrict__ out, int os,
-                                                                int ohs, int K, int N, HeadTail ht) {
+                                                                int ohs, int K, int N, HeadTail ht, HeadGate<TA> hg) {
   __shared__ float sx[HL_SMALL_K];
   __shared__ float red[4][64];
   const int t = blockIdx.x, h = blockIdx.y;
@@ -175,6 +187,7 @@ __global__ __launch_bounds__(256) void head_linear_small_kernel(const TA* __rest
   if (ht.positions) write_tail<TA>(ht, xr + K, out + (size_t)t * os + (size_t)h * ohs + N, t, threadIdx.x, blockDim.x);
   __syncthreads();
   const TA* Wh = W + (size_t)h * K * N;
+  const float gate = hg.at(t, h);
   const int per = (K + 3) >> 2;
   const int kb = wave * per, ke = min(K, kb + per);
   for (int n0 = 0; n0 < N; n0 += 64) {
@@ -191,14 +204,15 @@ __global__ __launch_bounds__(256) void head_linear_small_kernel(const TA* __rest
     __syncthreads();
     if (wave == 0 && n0 + lane < N)
       out[(size_t)t * os + (size_t)h * ohs + n0 + lane] =
-          from_float<TA>(((red[0][lane] + red[1][lane]) + red[2][lane]) + red[3][lane]);
+          from_float<TA>((((red[0][lane] + red[1][lane]) + red[2][lane]) + red[3][lane]) * gate);
     __syncthreads();
   }
 }
 
 extern "C" int sa_head_linear(const void* in, int is, int ihs, const void* W, void* out, int os, int ohs,
                               int act_dtype, int T, int H, int K, int N, const int* positions, const float* inv_freq,
-                              int rot, int tail, float magnitude, hipStream_t stream) {
+                              int rot, int tail, float magnitude, const void* gate, long long gate_stride,
+                              hipStream_t stream) {
   if (T <= 0) return 0;
   if (H <= 0 || K <= 0 || N <= 0 || H > 65535 || (N + 255) / 256 > 65535) return SA_ERR_ARG;
   if (positions && ((!inv_freq && rot > 0) || rot < 0 || (rot & 1) || tail < rot)) return SA_ERR_ARG;
@@ -207,10 +221,10 @@ extern "C" int sa_head_linear(const void* in, int is, int ihs, const void* W, vo
     dim3 grid(T, H), block(256);
     if (act_dtype == SA_F32)
       hipLaunchKernelGGL(head_linear_small_kernel<float>, grid, block, 0, stream, (const float*)in, is, ihs,
-                         (const float*)W, (float*)out, os, ohs, K, N, ht);
+                         (const float*)W, (float*)out, os, ohs, K, N, ht, HeadGate<float>{(const float*)gate, gate_stride});
     else if (act_dtype == SA_BF16)
       hipLaunchKernelGGL(head_linear_small_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)in, is, ihs,
-                         (const bf16_t*)W, (bf16_t*)out, os, ohs, K, N, ht);
+                         (const bf16_t*)W, (bf16_t*)out, os, ohs, K, N, ht, HeadGate<bf16_t>{(const bf16_t*)gate, gate_stride});
     else return SA_ERR_UNSUPPORTED;
     SA_LAUNCH_CHECK();
     return 0;
@@ -219,10 +233,10 @@ extern "C" int sa_head_linear(const void* in, int is, int ihs, const void* W, vo
   dim3 grid((T + HL_TT - 1) / HL_TT, H, (N + bx - 1) / bx), block(bx);
   if (act_dtype == SA_F32)
     hipLaunchKernelGGL(head_linear_kernel<float>, grid, block, 0, stream, (const float*)in, is, ihs, (const float*)W,
-                       (float*)out, os, ohs, T, K, N, ht);
+                       (float*)out, os, ohs, T, K, N, ht, HeadGate<float>{(const float*)gate, gate_stride});
   else if (act_dtype == SA_BF16)
     hipLaunchKernelGGL(head_linear_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)in, is, ihs,
-                       (const bf16_t*)W, (bf16_t*)out, os, ohs, T, K, N, ht);
+                       (const bf16_t*)W, (bf16_t*)out, os, ohs, T, K, N, ht, HeadGate<bf16_t>{(const bf16_t*)gate, gate_stride});
   else return SA_ERR_UNSUPPORTED;
   SA_LAUNCH_CHECK();
   return 0;

@@ -569,12 +569,13 @@ def delta_rule(z: torch.Tensor, conv_w: torch.Tensor, ba: torch.Tensor, A_log: t
 def latent_kv_write(z: torch.Tensor, norm_w: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor,
                     slots: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, eps: float, rank: int,
                     rot_dim: int, magnitude: float = 1.0) -> None:
-    """z [T, rank + rot_dim] -> the token's cache rows: k_pages [P, 1, page, Dp] gets
+    """z rows [T, rank + rot_dim] (a view with a row stride is fine) -> the token's cache rows: k_pages [P, 1, page, Dp] gets
     [normed latent | rotated key part | 0], v_pages [P, 1, Dp, page] the normed latent (and zeros).
     `magnitude` multiplies the rotation's sine and cosine."""
-    _dev(z, norm_w, positions, inv_freq, slots, k_pages, v_pages)
+    _dev(norm_w, positions, inv_freq, slots, k_pages, v_pages)
     T = z.shape[0]
-    _check(z.dim() == 2 and z.shape[1] == rank + rot_dim, f"z must be [T, {rank + rot_dim}]")
+    _rows(z, T, rank + rot_dim, "z")
+    _check(z.shape[1] == rank + rot_dim, f"z must be [T, {rank + rot_dim}]")
     P, one, page_size, Dp = k_pages.shape
     _check(one == 1 and Dp >= rank + rot_dim and v_pages.shape == (P, 1, Dp, page_size),
            "latent pages must be [P, 1, page, Dp] and [P, 1, Dp, page]")
@@ -586,18 +587,20 @@ def latent_kv_write(z: torch.Tensor, norm_w: torch.Tensor, positions: torch.Tens
     lib = load_library("latent")
     _ret(lib.sa_latent_kv_write(_ptr(z), c_int(_code(z)), _ptr(norm_w), _ptr(positions), _ptr(inv_freq), _ptr(slots),
                                 _ptr(k_pages), _ptr(v_pages), c_float(eps), c_int(T), c_int(rank), c_int(rot_dim),
-                                c_int(Dp), c_int(page_size), c_float(magnitude), _stream()), "latent_kv_write")
+                                c_int(Dp), c_int(page_size), c_float(magnitude), ctypes.c_longlong(z.stride(0)), _stream()),
+         "latent_kv_write")
 
 
 def head_linear(x: torch.Tensor, in_stride: int, in_head_stride: int, w: torch.Tensor, out: torch.Tensor,
                 out_stride: int, out_head_stride: int, T: int, positions: Optional[torch.Tensor] = None,
                 inv_freq: Optional[torch.Tensor] = None, rot: int = 0, tail: int = 0,
-                magnitude: float = 1.0) -> torch.Tensor:
+                magnitude: float = 1.0, gate_rows: Optional[torch.Tensor] = None, gate_col: int = 0) -> torch.Tensor:
     """out[t, h, :N] = x[t, h, :K] @ w[h] for w [H, K, N]: head h's K inputs of token t start at element
     t * in_stride + h * in_head_stride of x, its N outputs at t * out_stride + h * out_head_stride of out.
     With `positions`: behind the N outputs come the `rot` inputs that lie behind the head's K inputs, rotated by
     the token's position (dimension i with i + rot / 2, angles positions[t] * inv_freq[i], sine and cosine times
-    `magnitude`), then zeros up to `tail` places in all."""
+    `magnitude`), then zeros up to `tail` places in all.  With `gate_rows` (rows [T, >= gate_col + H] in x's dtype) a
+    head's N outputs are multiplied by sigmoid(gate_rows[t, gate_col + h])."""
     _dev(x, w, out, positions, inv_freq)
     _check(w.dim() == 3 and x.dtype == w.dtype == out.dtype, "head_linear: w must be [H, K, N], one dtype throughout")
     H, K, N = w.shape
@@ -611,11 +614,16 @@ def head_linear(x: torch.Tensor, in_stride: int, in_head_stride: int, w: torch.T
         _f32vec(inv_freq, rot // 2, "inv_freq")
         if T:
             _check(x.numel() >= (T - 1) * in_stride + (H - 1) * in_head_stride + K + rot, "head_linear: input too short")
+    gate, gs = c_void_p(0), 0
+    if gate_rows is not None:
+        _rows(gate_rows, T, gate_col + H, "gate rows")
+        _check(gate_rows.dtype == x.dtype and gate_col >= 0, "the gate's logits must have x's dtype")
+        gate, gs = c_void_p(gate_rows.data_ptr() + gate_col * gate_rows.element_size()), gate_rows.stride(0)
     lib = load_library("latent")
     _ret(lib.sa_head_linear(_ptr(x), c_int(in_stride), c_int(in_head_stride), _ptr(w), _ptr(out), c_int(out_stride),
                             c_int(out_head_stride), c_int(_code(x)), c_int(T), c_int(H), c_int(K), c_int(N),
                             _ptr(positions), _ptr(inv_freq), c_int(rot), c_int(tail), c_float(magnitude),
-                            _stream()), "head_linear")
+                            gate, ctypes.c_longlong(gs), _stream()), "head_linear")
     return out
 
 

@@ -115,12 +115,12 @@ class RoutedExperts(Part):
 
     def step_cost(self, tokens: int, context_before: int = 0) -> StepCost:
         """The router and the shared expert for every token; of the experts, `top` a token: their flops,
-        and as weights no more experts than the step's tokens can choose."""
+        and as weights no more experts than the step's tokens can choose (identity experts read and cost nothing; of a
+        token's choices as many are theirs as of the router's outputs, on the average)."""
         d, F = self.hidden_size, self.expert_size
-        used = min(self.experts, tokens * self.top)
+        used = min(self.experts, -(-tokens * self.top * self.experts // self.outputs))
         elements = self.outputs * d + used * 3 * F * d
         flops = 2.0 * tokens * self.outputs * d
-        # (identity experts cost nothing; of a token's choices as many are theirs as of the outputs, on the average)
         flops += 2.0 * tokens * self.top * (self.experts / self.outputs) * 3 * F * d
         if self.shared_size:
             elements += 3 * self.shared_size * d + (d if self.shared_gate else 0)

@@ -13,8 +13,8 @@ window and scale.
 
 Options: `q_rank`: the queries go through a latent of their own, q = W_uq (N(W_dq h) w_dq) (tensors `dq`, `dq.norm`,
 `uq` in place of `q`); `out_gate`: the concatenated heads are multiplied element by element with sigmoid(W_g h) before
-W_o, or (`out_gate="head"`) head h's output with the one number sigmoid(W_g h)_h, whose row of W_g rides behind the
-queries in their product.  The rotation of the shared key part may pair (i, i + rot_dim / 2) or (2i, 2i + 1): queries and keys are only ever
+W_o, or (`out_gate="head"`) head h's output with the one number sigmoid(W_g h)_h, which is
+applied where that output is made.  Without `q_rank` the queries, the heads' gate and the down-projection are one product.  The rotation of the shared key part may pair (i, i + rot_dim / 2) or (2i, 2i + 1): queries and keys are only ever
 multiplied with each other, so the second kind is the first after the rows of the projections that make the rotated
 parts have been put into the order (even places, odd places), which is done when the part loads.  A rotation with a
 magnitude (sine and cosine times a constant) is carried out by the kernels.
@@ -121,14 +121,6 @@ class LatentAttention(Part):
             self.q_norm = tensors["dq.norm"].float().contiguous()
         self.w_g = tensors["g"] if self.out_gate else None
         dt = self.wq.dtype
-        self.gate_col = -1                       # where the heads' gate logits lie behind the queries (-1: elsewhere)
-        if self.head_gate and not self.q_rank and tensors["g"].dtype == dt:
-            n = self.wq.shape[0] + H
-            pad = torch.zeros((-n % 8, self.hidden_size), dtype=dt, device=self.wq.device)       # (rows of whole vectors)
-            self.gate_col = self.wq.shape[0]
-            self.wq = torch.cat([self.wq, tensors["g"], pad], dim=0).contiguous()
-        elif self.head_gate:
-            self.w_g = tensors["g"]
         # [H, dim, R]: the queries' way into the latent space; [H, R, vdim]: the latents' way out
         self.w_uk = tensors["uk"].to(dt).view(H, self.dim, R).contiguous()
         self.w_uv = tensors["uv"].to(dt).view(H, self.vdim, R).transpose(1, 2).contiguous()
@@ -138,6 +130,22 @@ class LatentAttention(Part):
             if order is not None:
                 self.w_dkv = torch.cat([self.w_dkv[:R], self.w_dkv[R:][order]], dim=0).contiguous()
             self.latent_norm = tensors["dkv.norm"].float().contiguous()
+        if self.head_gate:
+            self.w_g = tensors["g"]
+        # one product of what reads the layer's input: queries | heads' gate | down-projection
+        self.w_in, self.cols = None, {}
+        together = [("q", self.wq)] if not self.q_rank else []
+        together += ([("g", self.w_g)] if self.head_gate else []) + ([("dkv", self.w_dkv)] if self.own_kv else [])
+        if not self.q_rank and self.head_gate and all(w.dtype == dt for _, w in together):
+            at = 0
+            for name, w in together:
+                self.cols[name] = at
+                at += w.shape[0]
+            pad = torch.zeros((-at % 8, self.hidden_size), dtype=dt, device=self.wq.device)       # (rows of whole vectors)
+            self.w_in = torch.cat([w for _, w in together] + [pad], dim=0).contiguous()
+            self.wq = self.w_g = self.w_dkv = None
+            _prepare_products(rt, self.w_in)
+            return
         _prepare_products(rt, self.wq)
 
     def forward(self, h: torch.Tensor, ctx, cache: LayerCache, writes_cache: bool = True) -> torch.Tensor:
@@ -148,13 +156,23 @@ class LatentAttention(Part):
         if k_pages.shape[-1] != D:
             raise ValueError(f"the cache keeps rows of {k_pages.shape[-1]}, this layer reads rows of {D}")
         with trace.span("write_to_cache"):
+            z = zin = gate = None
+            gate_col = 0
+            if self.w_in is not None:
+                zin = linear(h, self.w_in)
+                if self.own_kv:
+                    z = zin[:, self.cols["dkv"]: self.cols["dkv"] + R + self.rot_dim]
+                gate, gate_col = zin, self.cols["g"]
             if writes_cache:
                 if not self.own_kv:
                     raise ValueError("a latent attention without a down-projection cannot write a cache")
-                z = linear(h, self.w_dkv)
+                if z is None:
+                    z = linear(h, self.w_dkv)
                 ops.latent_kv_write(z, self.latent_norm, ctx.positions, self.inv_freq, grp.slots, k_pages, v_pages,
                                     self.eps, R, self.rot_dim, self.magnitude)
-            if self.q_rank:
+            if zin is not None:
+                q = zin                                                     # (the queries are its first columns)
+            elif self.q_rank:
                 # the queries' own latent: the product's fp32 sums are normed as a norm norms the stream
                 zq = linear(h, self.w_dq, out_dtype=torch.float32)
                 cq = ops.add_rmsnorm(zq, None, self.q_norm, self.eps, self.rt.empty((T, self.q_rank)))
@@ -169,11 +187,11 @@ class LatentAttention(Part):
         with trace.span("attention"):
             ops.paged_attention(qf, H * D, attn, k_pages, v_pages, grp.block_table, ctx, H, self.scale, self.window)
         o = self.rt.empty((T, H * self.vdim))
-        ops.head_linear(attn, H * D, D, self.w_uv, o, H * self.vdim, self.vdim, T)
+        if self.head_gate and gate is None:
+            gate = linear(h, self.w_g)
+        ops.head_linear(attn, H * D, D, self.w_uv, o, H * self.vdim, self.vdim, T, gate_rows=gate, gate_col=gate_col)
         if self.out_gate:
             ops.sigmoid_mul(o, linear(h, self.w_g))
-        elif self.head_gate:
-            ops.head_gate(o, *((q, self.gate_col) if self.gate_col >= 0 else (linear(h, self.w_g), 0)), H)
         return linear(o, self.wo, partial_ok=True)
 
 

@@ -348,6 +348,25 @@ def test_traces_through_the_program(tmp_path, dtype):
         bm.assert_matches_plain(torch.cat(rows[k]), folder, t, dtype, f"trace request {k}")
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_a_checkpoint_with_tensors_in_32_bit(tmp_path, dtype):
+    """Gates, corrections, norms and stream weights stored in float32 keep their precision in the bfloat16 engine (and
+    the products that put several matrices together are then made apart, or in float32)."""
+    from safetensors.torch import save_file
+    folder = bm.make_folder(tmp_path, "BA32", config=bm.BA, seed=3)
+    g = torch.Generator().manual_seed(1)
+    out = {}
+    for name, t in bm.plain_weights(folder).items():
+        if name.endswith((".g", ".correction", ".in", ".out", ".mix", ".norm1", ".norm2", ".b", ".conv")) and not name.endswith("mix.in"):
+            t = t.float() * (1 + 1e-3 * torch.randn(t.shape, generator=g))
+        out[name] = t.contiguous()
+    save_file(out, os.path.join(folder, "model.safetensors"))
+    engine = bm.engine_for(folder, dtype)
+    tokens = tokens_for(70, 15, bm.BA.vocab)
+    got = bm.run_portions(engine, "r", tokens, [40] + [1] * 20 + [10])
+    bm.assert_matches_plain(got, folder, tokens, dtype, "tensors in 32 bit")
+
+
 # ---------------------------------------------------------------------------------------------
 # the kernels alone
 # ---------------------------------------------------------------------------------------------
@@ -584,3 +603,32 @@ def test_embedding_in_copies(d, dtype):
     x = torch.empty((4, 3, d), dtype=torch.float32, device="cuda")
     ops.embed(E, tok, x, scale=2.0)
     assert torch.equal(x, (2.0 * E[tok.long()].float())[:, None].expand(4, 3, d))
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("T,H,K,N", [(1, 3, 40, 24), (7, 2, 96, 64), (64, 4, 24, 16), (65, 4, 24, 16), (300, 2, 130, 70)])
+def test_head_products_with_a_gate_per_head(dtype, T, H, K, N):
+    """Both kernels (few tokens and many), with the gate's logits in any column of a wider product, and the latent cache
+    write from a view of such a product."""
+    from serve_amd import ops
+    g = torch.Generator().manual_seed(T + K)
+    x = torch.randn(T, H * (K + 5), generator=g).to(dtype).cuda()
+    w = (torch.randn(H, K, N, generator=g) / K ** 0.5).to(dtype).cuda()
+    rows = torch.randn(T, 3 + H + 2, generator=g).to(dtype).cuda()
+    out = torch.empty((T, H * N), dtype=dtype, device="cuda")
+    ops.head_linear(x, H * (K + 5), K + 5, w, out, H * N, N, T, gate_rows=rows, gate_col=3)
+    xx = x.double().view(T, H, K + 5)[..., :K]
+    want = torch.stack([xx[:, h] @ w[h].double() for h in range(H)], dim=1) * torch.sigmoid(rows.double()[:, 3: 3 + H])[..., None]
+    tol = dict(atol=2e-5, rtol=2e-5) if dtype == torch.float32 else dict(atol=1e-2, rtol=1e-2)
+    assert torch.allclose(out.double().view(T, H, N), want, **tol)
+    R, dr, page, Dp = 20, 8, 4, 32
+    wide = torch.randn(T, R + dr + 11, generator=g).to(dtype).cuda()
+    nw = (1 + 0.1 * torch.randn(R, generator=g)).cuda()
+    pos = torch.arange(T, dtype=torch.int32, device="cuda")
+    P = -(-T // page)
+    pages = []
+    for z in (wide[:, 7: 7 + R + dr], wide[:, 7: 7 + R + dr].contiguous()):
+        k, v = torch.zeros((P, 1, page, Dp), dtype=dtype, device="cuda"), torch.zeros((P, 1, Dp, page), dtype=dtype, device="cuda")
+        ops.latent_kv_write(z, nw, pos, torch.ones(dr // 2, device="cuda"), pos, k, v, 1e-5, R, dr)
+        pages.append((k, v))
+    assert torch.equal(pages[0][0], pages[1][0]) and torch.equal(pages[0][1], pages[1][1]) and pages[0][0].abs().max() > 0
